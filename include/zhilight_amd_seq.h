@@ -42,6 +42,11 @@ int zls_version(void);
  * aligned, element loads otherwise. */
 int zls_gemm_nt(const void* x, int64_t ldx, const void* w, void* y, int64_t ldy, int64_t m, int64_t n, int64_t k, int dtype, int out_dtype,
                 zl_stream_t s);
+/* The same product with an epilogue: y = act(x . w^T + bias), bias fp32 (n) nullable, act -1 none, 0 relu(v)^2, 1 gelu_tanh(v), 2 silu(v),
+ * 3 softplus(v); y2 (nullable): the leading n2 columns of the result once more in `dtype` (rows of ldy2 >= n2 numbers) -- what a following
+ * product reads while the rest of y stays fp32. */
+int zls_gemm_nt_act(const void* x, int64_t ldx, const void* w, const float* bias, int act, void* y, int64_t ldy, void* y2, int64_t ldy2, int64_t n2,
+                    int64_t m, int64_t n, int64_t k, int dtype, int out_dtype, zl_stream_t s);
 /* The same with gathered rows: row r of x is x[x_rows[r]], row c of w is w[w_rows[c]] (device int32 arrays, NULL: in order; ldw: row
  * stride of w).  Always the tiled kernel.  The up-projection of cached rows that lie scattered over pages. */
 int zls_gemm_nt_gather(const void* x, int64_t ldx, const int32_t* x_rows, const void* w, int64_t ldw, const int32_t* w_rows, void* y,
@@ -113,19 +118,27 @@ int zls_latent_attention_prompt(const float* q, int64_t ldq, int64_t q_col0, con
 /* ---- state-space (Mamba-2) mixer ---------------------------------------------------------------------------------------------- */
 /* Causal per-channel convolution + SiLU over the columns col0 .. col0 + channels - 1 of proj: out[t][c] = silu(bias[c] + sum_k
  * w[c][k] * u[t - (taps - 1 - k)][c]); inputs before a portion's first token come from tail[slot] (taps - 1 rows, oldest first; zeros
- * for a new sequence).  zls_conv_tail_update then moves the portion's last taps - 1 inputs into tail[slot]; it must run after
- * zls_conv_silu on the same stream.  proj, out, tail fp32; w fp32 (channels, taps), bias fp32 (channels). */
-int zls_conv_silu(const float* proj, int64_t ld, int64_t col0, const float* w, const float* bias, const float* tail, int64_t channels,
+ * for a new sequence), and the portion's last taps - 1 inputs then replace them.  proj, out, tail fp32; w fp32 (channels, taps), bias fp32
+ * (channels). */
+int zls_conv_silu(const float* proj, int64_t ld, int64_t col0, const float* w, const float* bias, float* tail, int64_t channels,
                   int64_t taps, const zls_batch_t* b, float* out, zl_stream_t s);
-int zls_conv_tail_update(const float* proj, int64_t ld, int64_t col0, float* tail, int64_t channels, int64_t taps, const zls_batch_t* b,
-                         zl_stream_t s);
 /* The same convolution with its parts chosen: in_bias (nullable, fp32 (channels)) is added to every input u[t][c] before the taps (inputs
- * before a sequence's start stay 0; the tail holds inputs with the bias), bias (nullable) after them, act != 0 applies SiLU.
- * zls_short_conv_tail is its tail update (same in_bias). */
+ * before a sequence's start stay 0; the tail holds inputs with the bias), bias (nullable) after them, act != 0 applies SiLU; out_t
+ * (nullable): the result once more in `dtype`. */
 int zls_short_conv(const float* proj, int64_t ld, int64_t col0, const float* w, const float* bias, const float* in_bias, int act,
-                   const float* tail, int64_t channels, int64_t taps, const zls_batch_t* b, float* out, zl_stream_t s);
-int zls_short_conv_tail(const float* proj, int64_t ld, int64_t col0, const float* in_bias, float* tail, int64_t channels, int64_t taps,
-                        const zls_batch_t* b, zl_stream_t s);
+                   float* tail, int64_t channels, int64_t taps, const zls_batch_t* b, float* out, void* out_t, int dtype, zl_stream_t s);
+
+/* The selective recurrence with a decay per CHANNEL and state (Mamba): per channel c and state n, tokens in order,
+ *   S[n][c] <- 2^(dt_c a2[n][c]) S[n][c] + dt_c x_c B_n;   y_c = (sum_n S[n][c] C_n + d_c x_c) * silu(z_c)
+ * x, dt fp32 (n_tok, inner); B = bc[t][b_col0 ..], C = bc[t][c_col0 ..] (fp32 rows of ldbc numbers), z = zrow[t][z_col0 ..] (fp32 rows of
+ * ldz numbers); a2 fp32 (n_state, inner) = log2(e) times the (negative) rates; d fp32 (inner); state fp32 (slots, n_state, inner), read at
+ * the start and written back at the end; y (n_tok, inner) in `dtype`: the gated row, what the output projection reads.
+ * Portions above seg_len tokens (with a workspace of zls_selective_scan_workspace_bytes) run as segments in parallel: every segment from a
+ * zero state, the segments' start states, every segment again from its start state.  n_state <= 256. */
+int64_t zls_selective_scan_workspace_bytes(int64_t n_seq, int64_t max_count, int64_t seg_len, int64_t inner, int64_t n_state);
+int zls_selective_scan(const float* x, const float* dt, const float* bc, int64_t ldbc, int64_t b_col0, int64_t c_col0, const float* zrow, int64_t ldz,
+                       int64_t z_col0, const float* a2, const float* d, float* state, int64_t inner, int64_t n_state, const zls_batch_t* b, void* y,
+                       void* workspace, int64_t seg_len, int dtype, zl_stream_t s);
 
 /* The recurrence, one workgroup per (sequence, head), tokens in order:
  *   dt = softplus(dt_raw + dt_bias_h);  S <- exp(-exp(a_log_h) dt) S + dt B x^T;  y = S^T C + d_h x
@@ -169,6 +182,22 @@ int zls_add_layer_norm(float* x, const float* y, const float* w, const float* b,
 
 /* ---- softmax attention over a paged key / value cache: rotary positions, unit-RMS queries and keys, turned values, a sliding window,
  *      weights mixed across heads ------------------------------------------------------------------------------------------------- */
+/* The optional parts of zls_rope_norm_store (NULL: none of them):
+ *   whole_norm != 0: ALL heads * dim query numbers of a token are divided by ONE sqrt(mean of their squares + eps) before anything else, and
+ *   all kv_heads * dim key numbers by theirs, times q_w (heads * dim) / k_w (kv_heads * dim), fp32, nullable (qk_norm is 0 then);
+ *   temp_every > 0: the finished queries are multiplied by 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1);
+ *   x_heads > 0: x_heads more heads of x_dim numbers from column x_col0 of the same row are rotated in place, coordinate i < x_rot / 2 paired
+ *   with i + x_rot / 2, angle p * x_freq[i] (fp32 (x_rot / 2)) -- another mixer's queries and keys out of the same projection. */
+typedef struct {
+    int32_t whole_norm;
+    const float* q_w;
+    const float* k_w;
+    float temp_coef;
+    int32_t temp_every;
+    int32_t x_col0, x_heads, x_dim, x_rot;
+    const float* x_freq;
+} zls_head_prep_t;
+
 /* Per token at position p, in place on the fp32 projection row proj[t] (ld floats):
  *   queries (heads x dim from q_col0) and keys (kv_heads x dim from k_col0): coordinate i < rot_dims / 2 of a head is paired with
  *   i + rot_dims / 2 and the pair (u, v) becomes (u cos a - v sin a, v cos a + u sin a), a = p * qk_freq[i]; the other coordinates stay;
@@ -184,11 +213,12 @@ int zls_add_layer_norm(float* x, const float* y, const float* w, const float* b,
 int zls_rope_norm_store(float* proj, int64_t ld, int64_t q_col0, int64_t k_col0, int64_t v_col0, int64_t heads, int64_t kv_heads, int64_t dim,
                         int64_t vdim, const float* qk_freq, int64_t rot_dims, const float* v_freq, float eps, int qk_norm, int interleaved,
                         const float* vmix_src, int64_t vmix_ld, int64_t vmix_col0, float vmix_lambda, const float* q_norm_w, const float* k_norm_w,
-                        const zls_batch_t* b, void* k_cache, void* v_cache, int dtype, zl_stream_t s);
+                        const zls_head_prep_t* prep, const zls_batch_t* b, void* k_cache, void* v_cache, int dtype, zl_stream_t s);
 
 /* The optional score form of the two attention launches below (NULL: plain scaled scores and a softmax).  For query head g at position p
  * and key j:  s = scale * head_scale[g] * q.k;  s <- softcap * tanh(s / softcap) (softcap > 0);  s += bias[g][min(p - j, bias_rows - 1)];
  * chunk > 0: only keys with j / chunk == p / chunk are visible (chunks counted from position 0; not together with keep_first);
+ * slope: s -= slope[g] * (p - j), after the cap (a linear distance bias without an end);
  * sigmoid != 0: the weight of a visible key is sigmoid(s + offset[g]), every key on its own -- nothing is normalised, a split leaves
  * acc = sum_j w_j v_j and ml = (0, 1), and zls_head_mix_gate is called with plain_sum.  All pointers fp32 and nullable. */
 typedef struct {
@@ -199,6 +229,7 @@ typedef struct {
     const float* offset;       /* (heads) */
     int32_t chunk;
     int32_t sigmoid;
+    const float* slope;        /* (heads) */
 } zls_score_form_t;
 
 /* Softmax attention of every token over the cached keys j of its sequence with 0 <= p - j < window (window <= 0: all j <= p), and with
@@ -272,14 +303,15 @@ int zls_lowrank_decay(const float* proj, int64_t ld, int64_t u_col0, int64_t low
                       int64_t channels, int64_t n_tok, float* alpha, int dtype, zl_stream_t s);
 
 /* ---- mixture of experts over a ragged step ------------------------------------------------------------------------------------------ */
-/* Router: s = softmax(logits[t]) over all n_out outputs (score_kind 0) or sigmoid(logits[t][i]) of each (score_kind 1); choice = s +
- * correction (nullable); the outputs form `groups` equal groups of neighbours, a group's score is the sum of its `group_top` largest choice
+/* Router: s = softmax(logits[t]) over all n_out outputs (score_kind 0), sigmoid(logits[t][i]) of each (score_kind 1) or logits[t] (score_kind
+ * 2: the weights are then a softmax over the chosen logits only, renorm 0), the logits with logit_bias (fp32 (n_out), nullable) added; choice
+ * = s + correction (nullable); the outputs form `groups` equal groups of neighbours, a group's score is the sum of its `group_top` largest choice
  * scores (1: its largest), only outputs of the `keep` best groups can be chosen (groups <= 1: all) -- the others count as minus
  * infinity; the `top` largest choice scores are chosen (ties: the lower index).  ids int32 (n_tok, top), weights fp32 (n_tok, top) = s of
  * the chosen (divided by their sum + renorm_eps when renorm != 0), times weight_scale.  n_out <= 1024, n_out % groups == 0.  A token's
  * logits are the first n_out numbers of its row of ld >= n_out numbers. */
-int zls_moe_route(const float* logits, int64_t ld, int64_t n_tok, int64_t n_out, const float* correction, int64_t groups, int64_t keep, int64_t top,
-                  int renorm, int score_kind, int64_t group_top, float renorm_eps, float weight_scale, int32_t* ids, float* weights,
+int zls_moe_route(const float* logits, int64_t ld, int64_t n_tok, int64_t n_out, const float* logit_bias, const float* correction, int64_t groups,
+                  int64_t keep, int64_t top, int renorm, int score_kind, int64_t group_top, float renorm_eps, float weight_scale, int32_t* ids, float* weights,
                   zl_stream_t s);
 /* Sort the n_slots = n_tok * top (token, choice) pairs by expert: pairs whose id is >= n_experts (identity outputs) are left out.
  *   sorted_tok[p] = token of the pair at sorted position p;  slot_pos[t * top + k] = p (or -1);
@@ -301,13 +333,29 @@ int zls_gemm_nt_grouped(const void* x, int64_t ldx, const int32_t* x_rows, const
 int zls_silu_mul(const float* gu, int64_t rows, int64_t ff, void* out, int dtype, zl_stream_t s);
 /* out[p][c] = act(g, u) of gu fp32 (rows, 2 ff) in `dtype`: kind 0 silu(g) u; 1 gelu_tanh(g) u (tanh form); 2 g' sigmoid(alpha g') (u' + 1)
  * with g' = min(g, limit), u' = clamp(u, -limit, limit).  block 0: g = gu[p][c], u = gu[p][ff + c]; block > 0 (ff % block == 0): the row
- * holds blocks of `block` gates followed by their `block` ups (the packing of the gated grouped product). */
-int zls_act_mul(const float* gu, int64_t rows, int64_t ff, int kind, float alpha, float limit, int64_t block, void* out, int dtype,
+ * holds blocks of `block` gates followed by their `block` ups (the packing of the gated grouped product).  Rows of ld >= 2 ff numbers. */
+int zls_act_mul(const float* gu, int64_t ld, int64_t rows, int64_t ff, int kind, float alpha, float limit, int64_t block, void* out, int dtype,
                 zl_stream_t s);
 /* out[t] = sum_k weights[t][k] * (ids[t][k] >= n_experts ? h[t] : y[slot_pos[t * top + k]]), in the order of k; y fp32 (.., width),
- * h (n_tok, width) in `dtype`, out fp32. */
+ * h (n_tok, width) in `dtype`, out fp32.  shared (nullable, fp32 (n_tok, width)): a shared expert's rows, added last, times
+ * sigmoid(gate[t * ldg + g_col]) (gate nullable: times 1). */
 int zls_moe_combine(const float* y, const int32_t* slot_pos, const int32_t* ids, const float* weights, const void* h, int64_t n_tok,
-                    int64_t top, int64_t n_experts, int64_t width, float* out, int dtype, zl_stream_t s);
+                    int64_t top, int64_t n_experts, int64_t width, const float* shared, const float* gate, int64_t ldg, int64_t g_col, float* out,
+                    int dtype, zl_stream_t s);
+
+/* ---- sub-layers that run side by side ---------------------------------------------------------------------------------------------- */
+/* n <= 4 branch results y_i (fp32 (rows, width)) join the residual at once, and everything the next sub-layers read comes out of the same launch:
+ *   x[t] += sum_i coef_i * (w_i ? y_i / sqrt(mean(y_i^2) + eps) * w_i : y_i)        in place, the sum in the order of the branches; n may be 0
+ *   h1[t], h2[t] = x / sqrt(mean(x^2) + eps) * w1 | w2 of the NEW x in `dtype` (w1 / w2 nullable: two norms of one row share the mean)
+ *   xt[t * ldxt ..] = the new x once more in `dtype` (nullable)
+ * branches: host array; y, w, x fp32 device pointers.  width * 4 bytes <= 64 KiB. */
+typedef struct {
+    const float* y;
+    const float* w;
+    float coef;
+} zls_branch_t;
+int zls_add_branches(float* x, const zls_branch_t* branches, int64_t n, float eps, int64_t rows, int64_t width, const float* w1, void* h1,
+                     const float* w2, void* h2, void* xt, int64_t ldxt, int dtype, zl_stream_t s);
 
 /* ---- a residual kept as several streams ------------------------------------------------------------------------------------------ */
 /* The residual of a token is n <= 8 rows x_0 .. x_{n-1} of `width` fp32 numbers; element (t, s, i) of the streams that are READ lies at
@@ -323,7 +371,7 @@ int zls_streams_norm(const float* src, int64_t src_tok, int64_t src_stream, int6
 int zls_streams_update(const float* src, int64_t src_tok, int64_t src_stream, float* dst, int64_t n, const float* y, const float* gate,
                        int64_t ldg, int64_t g_col0, const float* gate_bias, const float* mix, const float* out_coef, const float* read_coef,
                        const float* w, float shift, float eps, int64_t n_tok, int64_t width, void* h, int dtype, zl_stream_t s);
-/* out[r][c] = act(z[r * ldz + c]) for fp32 z, out (rows, cols) in `dtype`: kind 0 relu(z)^2, 1 gelu_tanh(z), 2 silu(z). */
+/* out[r][c] = act(z[r * ldz + c]) for fp32 z, out (rows, cols) in `dtype`: kind 0 relu(z)^2, 1 gelu_tanh(z), 2 silu(z), 3 softplus(z). */
 int zls_unary_act(const float* z, int64_t ldz, int64_t rows, int64_t cols, int kind, void* out, int dtype, zl_stream_t s);
 
 #ifdef __cplusplus

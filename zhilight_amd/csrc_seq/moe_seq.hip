@@ -1,14 +1,15 @@
 // moe_seq.hip -- the routing side of a mixture-of-experts feed-forward over a ragged step (the products are zls_gemm_nt_grouped):
 //
-// k_moe_route    a wave per token: fp32 scores over all router outputs (softmax, or a sigmoid of each logit), choice scores = scores +
-//                correction, group-limited choice (a group's score = its best choice score, or the sum of its `group_top` best; outputs
+// k_moe_route    a wave per token: fp32 scores over all router outputs (softmax, a sigmoid of each logit, or the logits themselves -- then the
+//                weights are a softmax over the chosen ones --; the logits may get a bias first), choice scores = scores + correction, group-limited choice (a group's score = its best choice score, or the sum of its `group_top` best; outputs
 //                outside the best `keep` groups count as minus infinity), `top` picks by repeated arg-max (ties: the lower index),
 //                weights = the scores of the picks (optionally divided by their sum + renorm_eps), times weight_scale
 // k_moe_align    one workgroup: counts per expert, their prefix, every (token, choice) pair's place in the expert-sorted order, and the list of
 //                (expert, first, end) row tiles that the grouped product walks.  Identity outputs (id >= n_experts) take no place.
 // k_silu_mul     silu(gate) * up
 // k_act_mul      the gated activations of the feed-forwards: silu(g) u, gelu_tanh(g) u, or the clamped g sigmoid(a g) (u + 1)
-// k_moe_combine  a workgroup per token: the weighted sum of its picks' rows in the order of the picks; an identity pick adds the input row
+// k_moe_combine  a workgroup per token: the weighted sum of its picks' rows in the order of the picks; an identity pick adds the input row;
+//                a shared expert's row joins with a sigmoid gate per token
 #include "seq_common.h"
 
 namespace {
@@ -22,21 +23,25 @@ __device__ __forceinline__ void wave_argmax(float& v, int& i) {          // larg
     }
 }
 
-__global__ __launch_bounds__(64) void k_moe_route(const float* __restrict__ logits, int64_t ld, int n_out, const float* __restrict__ correction, int groups,
-                                                  int keep, int top, int renorm, int score_kind, int group_top, float renorm_eps,
+__global__ __launch_bounds__(64) void k_moe_route(const float* __restrict__ logits, int64_t ld, int n_out, const float* __restrict__ logit_bias,
+                                                  const float* __restrict__ correction, int groups, int keep, int top, int renorm, int score_kind, int group_top, float renorm_eps,
                                                   float weight_scale, int32_t* __restrict__ ids, float* __restrict__ weights) {
     __shared__ float prob[1024], choice[1024], gscore[1024];
     const int t = blockIdx.x, lane = threadIdx.x;
     const float* z = logits + (size_t)t * ld;                          // (the router's columns may lead wider rows)
     float mx = -INFINITY;
-    for (int i = lane; i < n_out; i += 64) mx = fmaxf(mx, z[i]);
+    auto logit = [&](int i) { return logit_bias ? z[i] + logit_bias[i] : z[i]; };
+    for (int i = lane; i < n_out; i += 64) mx = fmaxf(mx, logit(i));
     mx = zl_wave_max(mx);
     float sum = 0.f;
     if (score_kind == 1) {                                               // every output on its own: sigmoid of its logit
-        for (int i = lane; i < n_out; i += 64) prob[i] = seq_sigmoid(z[i]);
+        for (int i = lane; i < n_out; i += 64) prob[i] = seq_sigmoid(logit(i));
+        sum = 1.0f;
+    } else if (score_kind == 2) {                                        // the choice is among the logits themselves (softmax over the chosen: below)
+        for (int i = lane; i < n_out; i += 64) prob[i] = logit(i);
         sum = 1.0f;
     } else {
-        for (int i = lane; i < n_out; i += 64) { const float e = expf(z[i] - mx); prob[i] = e; sum += e; }
+        for (int i = lane; i < n_out; i += 64) { const float e = expf(logit(i) - mx); prob[i] = e; sum += e; }
         sum = zl_wave_sum(sum);
     }
     for (int i = lane; i < n_out; i += 64) {
@@ -99,6 +104,17 @@ __global__ __launch_bounds__(64) void k_moe_route(const float* __restrict__ logi
         }
         wsum += prob[bi];
         __syncthreads();
+    }
+    if (score_kind == 2) {                                               // weights: a softmax over the chosen logits only (the first pick is the
+        __syncthreads();                                                 // largest unless a correction moved the choice)
+        float m = -INFINITY;
+        for (int k = lane; k < top; k += 64) m = fmaxf(m, weights[(size_t)t * top + k]);
+        m = zl_wave_max(m);
+        float l = 0.f;
+        for (int k = lane; k < top; k += 64) l += expf(weights[(size_t)t * top + k] - m);
+        l = zl_wave_sum(l);
+        for (int k = lane; k < top; k += 64) weights[(size_t)t * top + k] = expf(weights[(size_t)t * top + k] - m) / l * weight_scale;
+        return;
     }
     if (renorm || weight_scale != 1.0f) {
         __syncthreads();
@@ -178,20 +194,22 @@ __global__ __launch_bounds__(256) void k_silu_mul(const float* __restrict__ gu, 
 
 // block > 0: the row holds blocks of `block` gate columns followed by their `block` up columns; 0: all gates, then all ups
 template <int DT>
-__global__ __launch_bounds__(256) void k_act_mul(const float* __restrict__ gu, int ff, int kind, float alpha, float limit, int block,
+__global__ __launch_bounds__(256) void k_act_mul(const float* __restrict__ gu, int64_t ld, int ff, int kind, float alpha, float limit, int block,
                                                  void* __restrict__ out) {
     const size_t r = blockIdx.x;
     for (int c = threadIdx.x; c < ff; c += 256) {
         const int gi = block > 0 ? (c / block) * 2 * block + c % block : c, ui = block > 0 ? gi + block : ff + c;
-        SeqT<DT>::st(out, r * ff + c, gated_act(gu[r * 2 * ff + gi], gu[r * 2 * ff + ui], kind, alpha, limit));
+        SeqT<DT>::st(out, r * ff + c, gated_act(gu[r * ld + gi], gu[r * ld + ui], kind, alpha, limit));
     }
 }
 
 template <int DT>
 __global__ __launch_bounds__(256) void k_moe_combine(const float* __restrict__ y, const int32_t* __restrict__ slot_pos, const int32_t* __restrict__ ids,
                                                      const float* __restrict__ weights, const void* __restrict__ h, int top, int n_experts, int width,
+                                                     const float* __restrict__ shared, const float* __restrict__ gate, int64_t ldg, int g_col,
                                                      float* __restrict__ out) {
     const size_t t = blockIdx.x;
+    const float sg = shared ? (gate ? seq_sigmoid(gate[t * ldg + g_col]) : 1.0f) : 0.f;
     for (int c = threadIdx.x; c < width; c += 256) {
         float a = 0.f;
         for (int k = 0; k < top; ++k) {
@@ -200,21 +218,22 @@ __global__ __launch_bounds__(256) void k_moe_combine(const float* __restrict__ y
             const float v = e >= n_experts ? SeqT<DT>::ld(h, t * width + c) : y[(size_t)slot_pos[t * top + k] * width + c];
             a = fmaf(w, v, a);
         }
+        if (shared) a = fmaf(sg, shared[t * width + c], a);
         out[t * width + c] = a;
     }
 }
 
 }  // namespace
 
-extern "C" int zls_moe_route(const float* logits, int64_t ld, int64_t n_tok, int64_t n_out, const float* correction, int64_t groups, int64_t keep, int64_t top,
+extern "C" int zls_moe_route(const float* logits, int64_t ld, int64_t n_tok, int64_t n_out, const float* logit_bias, const float* correction, int64_t groups, int64_t keep, int64_t top,
                              int renorm, int score_kind, int64_t group_top, float renorm_eps, float weight_scale, int32_t* ids, float* weights,
                              zl_stream_t s) {
     ZL_CHECK_ARG(logits && ids && weights && n_tok > 0 && n_out > 0 && top > 0 && ld >= n_out, ZL_EINVAL);
     ZL_CHECK_ARG(n_out <= 1024 && top <= n_out, ZL_ELIMIT);
     if (groups < 1) groups = 1;
     ZL_CHECK_ARG(n_out % groups == 0 && keep >= 1 && keep <= groups && top <= keep * (n_out / groups), ZL_ESHAPE);
-    ZL_CHECK_ARG((score_kind == 0 || score_kind == 1) && group_top >= 1, ZL_EINVAL);
-    hipLaunchKernelGGL(k_moe_route, dim3((unsigned)n_tok), dim3(64), 0, (hipStream_t)s, logits, ld, (int)n_out, correction, (int)groups, (int)keep,
+    ZL_CHECK_ARG(score_kind >= 0 && score_kind <= 2 && !(score_kind == 2 && renorm) && group_top >= 1, ZL_EINVAL);
+    hipLaunchKernelGGL(k_moe_route, dim3((unsigned)n_tok), dim3(64), 0, (hipStream_t)s, logits, ld, (int)n_out, logit_bias, correction, (int)groups, (int)keep,
                        (int)top, renorm, score_kind, (int)group_top, renorm_eps, weight_scale, ids, weights);
     return zl_launch_status();
 }
@@ -238,20 +257,22 @@ extern "C" int zls_silu_mul(const float* gu, int64_t rows, int64_t ff, void* out
     return zl_launch_status();
 }
 
-extern "C" int zls_act_mul(const float* gu, int64_t rows, int64_t ff, int kind, float alpha, float limit, int64_t block, void* out, int dtype,
+extern "C" int zls_act_mul(const float* gu, int64_t ld, int64_t rows, int64_t ff, int kind, float alpha, float limit, int64_t block, void* out, int dtype,
                            zl_stream_t s) {
-    ZL_CHECK_ARG(gu && out && rows > 0 && ff > 0 && kind >= 0 && kind <= 2 && block >= 0 && (block == 0 || ff % block == 0), ZL_EINVAL);
-#define CALL(DT) hipLaunchKernelGGL((k_act_mul<DT>), dim3((unsigned)rows), dim3(256), 0, (hipStream_t)s, gu, (int)ff, kind, alpha, limit, (int)block, out);
+    ZL_CHECK_ARG(gu && out && rows > 0 && ff > 0 && kind >= 0 && kind <= 2 && block >= 0 && (block == 0 || ff % block == 0) && ld >= 2 * ff, ZL_EINVAL);
+#define CALL(DT) hipLaunchKernelGGL((k_act_mul<DT>), dim3((unsigned)rows), dim3(256), 0, (hipStream_t)s, gu, ld, (int)ff, kind, alpha, limit, (int)block, out);
     ZLS_DISPATCH(dtype, CALL)
 #undef CALL
     return zl_launch_status();
 }
 
 extern "C" int zls_moe_combine(const float* y, const int32_t* slot_pos, const int32_t* ids, const float* weights, const void* h, int64_t n_tok,
-                               int64_t top, int64_t n_experts, int64_t width, float* out, int dtype, zl_stream_t s) {
+                               int64_t top, int64_t n_experts, int64_t width, const float* shared, const float* gate, int64_t ldg, int64_t g_col,
+                               float* out, int dtype, zl_stream_t s) {
+    ZL_CHECK_ARG(!gate || (shared && g_col >= 0 && g_col < ldg), ZL_EINVAL);
     ZL_CHECK_ARG(y && slot_pos && ids && weights && h && out && n_tok > 0 && top > 0 && width > 0, ZL_EINVAL);
 #define CALL(DT) hipLaunchKernelGGL((k_moe_combine<DT>), dim3((unsigned)n_tok), dim3(256), 0, (hipStream_t)s, y, slot_pos, ids, weights, h, (int)top, \
-                                    (int)n_experts, (int)width, out);
+                                    (int)n_experts, (int)width, shared, gate, ldg, (int)g_col, out);
     ZLS_DISPATCH(dtype, CALL)
 #undef CALL
     return zl_launch_status();

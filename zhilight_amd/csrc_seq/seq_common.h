@@ -30,6 +30,13 @@ __device__ __forceinline__ float gated_act(float g, float u, int kind, float alp
     }
     return seq_silu(g) * u;
 }
+// the activations of ungated feed-forwards and of a product's epilogue: 0 relu(v)^2, 1 gelu_tanh(v), 2 silu(v), 3 softplus(v)
+__device__ __forceinline__ float unary_act(float v, int kind) {
+    if (kind == 0) { const float m = fmaxf(v, 0.f); return m * m; }
+    if (kind == 1) return 0.5f * v * (1.0f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v)));
+    if (kind == 2) return seq_silu(v);
+    return seq_softplus(v);
+}
 // sine and cosine of an fp32 angle of any size (positions times frequencies reach thousands of radians): the angle is brought into
 // [-pi, pi] in double (exact to 1e-9 for angles up to 2^24), where the fp32 functions take their short path
 __device__ __forceinline__ void seq_sincos(float a, float* sn, float* cs) {

@@ -2,7 +2,8 @@
 // its carried row, the scalar-gain RMS norm fused with the residual sum, the gathered final norm, PolyNorm, layer norm, the weighted RMS
 // norm before a sub-layer (alone, or fused with the residual sum that precedes it), scaled and soft-capped logits, and the same two steps
 // for a residual kept as SEVERAL streams (k_streams_norm, k_streams_update): a sub-layer reads a weighted sum of the streams, its result --
-// optionally gated by a sigmoid -- goes to every stream with a factor of its own while the streams are mixed by a small matrix.
+// optionally gated by a sigmoid -- goes to every stream with a factor of its own while the streams are mixed by a small matrix -- and for
+// sub-layers that run side by side (k_add_branches: normed or plain results join the residual together, two norms of the new row come out).
 // One workgroup per token row; every sum of squares is fp32 (butterfly inside a wave, waves in order).
 #include "seq_common.h"
 
@@ -160,6 +161,95 @@ __global__ __launch_bounds__(kT) void k_add_rms_norm(float* __restrict__ x, cons
     for (int i = threadIdx.x; i < width; i += kT) SeqT<DT>::st(h2, row + i, x[row + i] * f * (w2[i] + shift));
 }
 
+// V consecutive fp32 numbers (V = 4: one 16-byte access)
+template <int V> struct VecF;
+template <> struct VecF<1> {
+    static __device__ __forceinline__ void ld(const float* p, float* v) { v[0] = *p; }
+    static __device__ __forceinline__ void st(float* p, const float* v) { *p = v[0]; }
+};
+template <> struct VecF<4> {
+    static __device__ __forceinline__ void ld(const float* p, float* v) {
+        const float4 a = *reinterpret_cast<const float4*>(p);
+        v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w;
+    }
+    static __device__ __forceinline__ void st(float* p, const float* v) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
+};
+
+constexpr int kMaxBranches = 4;
+
+struct BranchP {
+    float* x;
+    const float* y[kMaxBranches]; const float* w[kMaxBranches]; float coef[kMaxBranches];
+    float eps; int width;
+    const float* w1; void* h1; const float* w2; void* h2;
+    void* xt; int64_t ldxt;
+};
+
+// x += sum_i coef_i N_i(y_i) of NB branches that ran side by side, and the inputs of the next two sub-layers, both norms of the same new
+// row.  The new row stays in LDS between its sum of squares and its norms; a normed branch is read twice, the second time from L2.
+template <int DT, int NB, int V>
+__global__ __launch_bounds__(kT) void k_add_branches(const BranchP p) {
+    extern __shared__ __attribute__((aligned(16))) float u[];
+    __shared__ float red[16];
+    const size_t row = (size_t)blockIdx.x * p.width;
+    float ss[NB > 0 ? NB : 1];
+    bool any = false;
+#pragma unroll
+    for (int b = 0; b < NB; ++b) { ss[b] = 0.f; any = any || p.w[b] != nullptr; }
+    if (any)
+        for (int i = threadIdx.x * V; i < p.width; i += kT * V)
+#pragma unroll
+            for (int b = 0; b < NB; ++b)
+                if (p.w[b]) {
+                    float v[V];
+                    VecF<V>::ld(p.y[b] + row + i, v);
+#pragma unroll
+                    for (int e = 0; e < V; ++e) ss[b] = fmaf(v[e], v[e], ss[b]);
+                }
+    float f[NB > 0 ? NB : 1];
+#pragma unroll
+    for (int b = 0; b < NB; ++b) f[b] = p.w[b] ? p.coef[b] / sqrtf(zl_block_sum(ss[b], red) / (float)p.width + p.eps) : p.coef[b];
+    float sx = 0.f;
+    for (int i = threadIdx.x * V; i < p.width; i += kT * V) {
+        float x[V];
+        VecF<V>::ld(p.x + row + i, x);
+        if (NB > 0) {
+            float a[V];
+#pragma unroll
+            for (int e = 0; e < V; ++e) a[e] = 0.f;
+#pragma unroll
+            for (int b = 0; b < NB; ++b) {
+                float v[V];
+                VecF<V>::ld(p.y[b] + row + i, v);
+                if (p.w[b]) {
+                    float w[V];
+                    VecF<V>::ld(p.w[b] + i, w);
+#pragma unroll
+                    for (int e = 0; e < V; ++e) v[e] *= w[e];
+                }
+#pragma unroll
+                for (int e = 0; e < V; ++e) a[e] = fmaf(f[b], v[e], a[e]);
+            }
+#pragma unroll
+            for (int e = 0; e < V; ++e) x[e] += a[e];
+            VecF<V>::st(p.x + row + i, x);
+        }
+        VecF<V>::st(u + i, x);
+#pragma unroll
+        for (int e = 0; e < V; ++e) {
+            sx = fmaf(x[e], x[e], sx);
+            if (p.xt) SeqT<DT>::st(p.xt, (size_t)blockIdx.x * p.ldxt + i + e, x[e]);
+        }
+    }
+    if (!p.w1 && !p.w2) return;
+    const float fx = 1.0f / sqrtf(zl_block_sum(sx, red) / (float)p.width + p.eps);
+    for (int i = threadIdx.x; i < p.width; i += kT) {
+        const float v = u[i] * fx;
+        if (p.w1) SeqT<DT>::st(p.h1, row + i, v * p.w1[i]);
+        if (p.w2) SeqT<DT>::st(p.h2, row + i, v * p.w2[i]);
+    }
+}
+
 // z <- cap * tanh(z * scale / cap) (cap <= 0: z * scale)
 __global__ __launch_bounds__(kT) void k_scale_softcap(float* __restrict__ z, int64_t n, float scale, float cap) {
     const int64_t i = (int64_t)blockIdx.x * kT + threadIdx.x;
@@ -206,20 +296,6 @@ __global__ __launch_bounds__(kT) void k_streams_norm(const StreamsP p) {
     const float f = 1.0f / sqrtf(zl_block_sum(ss, red) / (float)p.width + p.eps);
     for (int i = threadIdx.x; i < p.width; i += kT) SeqT<DT>::st(p.h, (size_t)blockIdx.x * p.width + i, u[i] * f * (p.w[i] + p.shift));
 }
-
-// V consecutive fp32 numbers (V = 4: one 16-byte access)
-template <int V> struct VecF;
-template <> struct VecF<1> {
-    static __device__ __forceinline__ void ld(const float* p, float* v) { v[0] = *p; }
-    static __device__ __forceinline__ void st(float* p, const float* v) { *p = v[0]; }
-};
-template <> struct VecF<4> {
-    static __device__ __forceinline__ void ld(const float* p, float* v) {
-        const float4 a = *reinterpret_cast<const float4*>(p);
-        v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w;
-    }
-    static __device__ __forceinline__ void st(float* p, const float* v) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
-};
 
 // x_t <- sum_s mix[s][t] x_s + out_coef[t] * y * sigmoid(gate + bias), all streams from the old ones (a thread holds its elements of every
 // stream in registers before it writes); with read_coef also the NEXT sub-layer's input, the normed weighted sum of the new streams.
@@ -278,7 +354,7 @@ __global__ __launch_bounds__(kT) void k_streams_update(const StreamsP p) {
     for (int i = threadIdx.x; i < p.width; i += kT) SeqT<DT>::st(p.h, t * p.width + i, u[i] * f * (p.w[i] + p.shift));
 }
 
-// out = act(z): kind 0 relu(z)^2, 1 gelu_tanh(z), 2 silu(z); V consecutive elements of a row per thread
+// out = act(z) (unary_act in seq_common.h); V consecutive elements of a row per thread
 template <int DT, int V>
 __global__ __launch_bounds__(kT) void k_unary_act(const float* __restrict__ z, int64_t ldz, int64_t rows, int64_t cols, int kind, void* __restrict__ out) {
     const int64_t e = ((int64_t)blockIdx.x * kT + threadIdx.x) * V;
@@ -287,11 +363,7 @@ __global__ __launch_bounds__(kT) void k_unary_act(const float* __restrict__ z, i
     VecF<V>::ld(z + (e / cols) * ldz + e % cols, v);
 #pragma unroll
     for (int i = 0; i < V; ++i) {
-        float r;
-        if (kind == 0) { const float m = fmaxf(v[i], 0.f); r = m * m; }
-        else if (kind == 1) r = 0.5f * v[i] * (1.0f + tanhf(0.7978845608028654f * (v[i] + 0.044715f * v[i] * v[i] * v[i])));
-        else r = seq_silu(v[i]);
-        SeqT<DT>::st(out, (size_t)e + i, r);
+        SeqT<DT>::st(out, (size_t)e + i, unary_act(v[i], kind));
     }
 }
 
@@ -385,6 +457,35 @@ extern "C" int zls_scale_softcap(float* z, int64_t n, float scale, float cap, zl
     return zl_launch_status();
 }
 
+extern "C" int zls_add_branches(float* x, const zls_branch_t* branches, int64_t n, float eps, int64_t rows, int64_t width, const float* w1, void* h1,
+                                const float* w2, void* h2, void* xt, int64_t ldxt, int dtype, zl_stream_t s) {
+    ZL_CHECK_ARG(x && rows > 0 && width > 0 && n >= 0 && (n == 0 || branches) && (!w1 || h1) && (!w2 || h2) && (!xt || ldxt >= width), ZL_EINVAL);
+    ZL_CHECK_ARG(n <= kMaxBranches && width * sizeof(float) <= 60 * 1024, ZL_ELIMIT);
+    BranchP p = {};
+    auto al = [](const void* q) { return ((uintptr_t)q & 15) == 0; };
+    bool vec = width % 4 == 0 && al(x);
+    for (int i = 0; i < n; ++i) {
+        ZL_CHECK_ARG(branches[i].y, ZL_EINVAL);
+        p.y[i] = branches[i].y; p.w[i] = branches[i].w; p.coef[i] = branches[i].coef;
+        vec = vec && al(p.y[i]) && al(p.w[i]);
+    }
+    p.x = x; p.eps = eps; p.width = (int)width; p.w1 = w1; p.h1 = h1; p.w2 = w2; p.h2 = h2; p.xt = xt; p.ldxt = ldxt;
+    const dim3 grid((unsigned)rows);
+    const size_t lds = (size_t)(width + 3) / 4 * 16;
+    hipStream_t hs = (hipStream_t)s;
+#define GO(DT, NB)                                                                                 \
+    if (vec) hipLaunchKernelGGL((k_add_branches<DT, NB, 4>), grid, dim3(kT), lds, hs, p);          \
+    else hipLaunchKernelGGL((k_add_branches<DT, NB, 1>), grid, dim3(kT), lds, hs, p);
+#define CALL(DT)                                                                                   \
+    switch (n) {                                                                                   \
+        case 0: GO(DT, 0) break; case 1: GO(DT, 1) break; case 2: GO(DT, 2) break; case 3: GO(DT, 3) break; default: GO(DT, 4) break; \
+    }
+    ZLS_DISPATCH(dtype, CALL)
+#undef CALL
+#undef GO
+    return zl_launch_status();
+}
+
 extern "C" int zls_streams_norm(const float* src, int64_t src_tok, int64_t src_stream, int64_t n, const float* read_coef, const int32_t* rows,
                                 const float* w, float shift, float eps, int64_t n_rows, int64_t width, void* h, int dtype, zl_stream_t s) {
     ZL_CHECK_ARG(src && w && h && n_rows > 0 && width > 0 && n > 0 && src_tok >= 0 && src_stream >= 0, ZL_EINVAL);
@@ -430,7 +531,7 @@ extern "C" int zls_streams_update(const float* src, int64_t src_tok, int64_t src
 }
 
 extern "C" int zls_unary_act(const float* z, int64_t ldz, int64_t rows, int64_t cols, int kind, void* out, int dtype, zl_stream_t s) {
-    ZL_CHECK_ARG(z && out && rows > 0 && cols > 0 && ldz >= cols && kind >= 0 && kind <= 2, ZL_EINVAL);
+    ZL_CHECK_ARG(z && out && rows > 0 && cols > 0 && ldz >= cols && kind >= 0 && kind <= 3, ZL_EINVAL);
     const int64_t n = rows * cols;
     ZL_CHECK_ARG(n < (1LL << 40), ZL_ELIMIT);
     const bool vec = cols % 4 == 0 && ldz % 4 == 0 && ((uintptr_t)z & 15) == 0;

@@ -9,6 +9,7 @@
 //   k_seq_gemm  more rows (prompt portions, mixed steps): 128 x 128 or 64 x 64 output tile per workgroup of 4 waves (2 x 2; a wave =
 //               4 x 4 or 2 x 2 MFMA tiles of 16 x 16), 32-k slices of x and W staged through LDS (zero-filled past the edges), the next slice's global
 //               loads issued before the current slice's MFMAs.  bf16: v_mfma_f32_16x16x32_bf16; fp32: v_mfma_f32_16x16x4_f32.
+// Each has an instantiation with an epilogue (EPI: bias, activation, leading columns once more in the serving format).
 #include "seq_common.h"
 
 namespace {
@@ -29,7 +30,21 @@ struct GemmP {
     const int32_t* tiles;
     int64_t w_stride;
     int act; float act_alpha, act_limit;                       // the gated epilogue's activation (gated_act in seq_common.h)
+    // the epilogue of EPI instantiations: y = unary_act(x . w^T + bias, uact) (bias nullable; uact < 0: no activation), and the leading n2
+    // columns once more in the format of x to y2 (nullable): what a following product reads while the rest stays fp32
+    const float* bias; int uact;
+    void* y2; int64_t ldy2; int n2;
 };
+
+template <int DT, int ODT, bool EPI>
+__device__ __forceinline__ void put(const GemmP& p, int row, int col, float v) {
+    if constexpr (EPI) {
+        if (p.bias) v += p.bias[col];
+        if (p.uact >= 0) v = unary_act(v, p.uact);
+        if (col < p.n2) SeqT<DT>::st(p.y2, (size_t)row * p.ldy2 + col, v);
+    }
+    SeqT<ODT>::st(p.y, (size_t)row * p.ldy + col, v);
+}
 
 // ---- tiles in LDS -----------------------------------------------------------------------------------------------------------------
 template <int DT> struct Tile;
@@ -73,7 +88,7 @@ template <> struct Tile<ZL_F32> {
 // WT x WT MFMA tiles per wave: the workgroup's output tile is (32 WT) x (32 WT)
 // GATED: the weight rows come in blocks of 16 gate rows followed by their 16 up rows, so that a wave's even column tiles are gates and the
 // odd ones the up projections of the same 16 outputs; the epilogue writes act(gate, up) (gated_act: silu(gate) * up and others), half as many columns
-template <int DT, int ODT, int WT, bool GATED = false>
+template <int DT, int ODT, int WT, bool GATED = false, bool EPI = false>
 __global__ __launch_bounds__(256) void k_seq_gemm(const GemmP p) {
     typedef typename Tile<DT>::elem E;
     constexpr int RS = Tile<DT>::kRow;
@@ -180,7 +195,7 @@ __global__ __launch_bounds__(256) void k_seq_gemm(const GemmP p) {
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int row = m0 + wm * 16 * WT + i * 16 + 4 * kq + r;
-                if (row < mlim && col < p.n) SeqT<ODT>::st(p.y, (size_t)row * p.ldy + col, acc[i][j][r]);
+                if (row < mlim && col < p.n) put<DT, ODT, EPI>(p, row, col, acc[i][j][r]);
             }
         }
 }
@@ -208,7 +223,7 @@ template <> struct Vec8<ZL_F32> {
 
 // CPW output columns per wave: the activation rows (L2) are read once per CPW weight rows (HBM) -- with 8 rows and one column per wave
 // the activations would be eight times the weight traffic
-template <int DT, int ODT, int MR, int CPW>
+template <int DT, int ODT, int MR, int CPW, bool EPI = false>
 __global__ __launch_bounds__(256) void k_seq_gemv(const GemmP p) {
     const int lane = threadIdx.x & 63;
     const int col0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * CPW;
@@ -257,7 +272,7 @@ __global__ __launch_bounds__(256) void k_seq_gemv(const GemmP p) {
 #pragma unroll
         for (int c = 0; c < CPW; ++c) {
             const float v = zl_wave_sum(acc[r][c]);
-            if (lane == 0 && r < p.m && col0 + c < p.n) SeqT<ODT>::st(p.y, (size_t)r * p.ldy + col0 + c, v);
+            if (lane == 0 && r < p.m && col0 + c < p.n) put<DT, ODT, EPI>(p, r, col0 + c, v);
         }
 }
 
@@ -266,7 +281,7 @@ __global__ __launch_bounds__(256) void k_seq_gemv(const GemmP p) {
 // activation row (B operand: lane = row; rows past m are zero), eight steps in flight, one v_mfma_f32_16x16x32_bf16 each.  The weights are
 // read exactly once, the activations cost half the weight bytes at 8 rows (L2), and no VALU multiply is spent.  The four partial tiles
 // meet in LDS.
-template <int ODT>
+template <int ODT, bool EPI = false>
 __global__ __launch_bounds__(256) void k_seq_gemv_mfma(const GemmP p) {
     __shared__ float red[4][16][17];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nrow = lane & 15, kq = lane >> 4;
@@ -295,7 +310,7 @@ __global__ __launch_bounds__(256) void k_seq_gemv_mfma(const GemmP p) {
     __syncthreads();
     const int c = threadIdx.x >> 4, m = threadIdx.x & 15;
     if (m < p.m && col0 + c < p.n)
-        SeqT<ODT>::st(p.y, (size_t)m * p.ldy + col0 + c, red[0][c][m] + red[1][c][m] + red[2][c][m] + red[3][c][m]);
+        put<ZL_BF16, ODT, EPI>(p, m, col0 + c, red[0][c][m] + red[1][c][m] + red[2][c][m] + red[3][c][m]);
 }
 
 // the grouped product for a FEW rows (decode steps of a mixture of experts): a wave per (sorted row, output column) streams the column's
@@ -339,32 +354,32 @@ __global__ __launch_bounds__(256) void k_seq_gemv_grouped(const GemmP p, const i
 }
 
 // 128 x 128 tiles (four times the MFMAs per LDS fragment) when they still fill the chip, 64 x 64 otherwise
-template <int DT, int ODT>
+template <int DT, int ODT, bool EPI = false>
 void launch_tiled(const GemmP& p, hipStream_t hs) {
     const int64_t big = (int64_t)((p.m + 127) / 128) * ((p.n + 127) / 128);
     if (big >= 256) {
         const dim3 grid((unsigned)((p.n + 127) / 128), (unsigned)((p.m + 127) / 128));
-        hipLaunchKernelGGL((k_seq_gemm<DT, ODT, 4>), grid, dim3(256), 0, hs, p);
+        hipLaunchKernelGGL((k_seq_gemm<DT, ODT, 4, false, EPI>), grid, dim3(256), 0, hs, p);
     } else {
         const dim3 grid((unsigned)((p.n + 63) / 64), (unsigned)((p.m + 63) / 64));
-        hipLaunchKernelGGL((k_seq_gemm<DT, ODT, 2>), grid, dim3(256), 0, hs, p);
+        hipLaunchKernelGGL((k_seq_gemm<DT, ODT, 2, false, EPI>), grid, dim3(256), 0, hs, p);
     }
 }
 
-template <int DT, int ODT>
+template <int DT, int ODT, bool EPI = false>
 int launch(const GemmP& p, hipStream_t hs) {
     if constexpr (DT == ZL_BF16) {
         if (p.m >= 3 && p.m <= 16 && p.vec && (p.k & 7) == 0) {
-            hipLaunchKernelGGL((k_seq_gemv_mfma<ODT>), dim3((unsigned)((p.n + 15) / 16)), dim3(256), 0, hs, p);
+            hipLaunchKernelGGL((k_seq_gemv_mfma<ODT, EPI>), dim3((unsigned)((p.n + 15) / 16)), dim3(256), 0, hs, p);
             return zl_launch_status();
         }
     }
     if (p.m <= 8) {
-        if (p.m <= 2) hipLaunchKernelGGL((k_seq_gemv<DT, ODT, 2, 1>), dim3((unsigned)((p.n + 3) / 4)), dim3(256), 0, hs, p);
-        else if (p.m <= 4) hipLaunchKernelGGL((k_seq_gemv<DT, ODT, 4, 2>), dim3((unsigned)((p.n + 7) / 8)), dim3(256), 0, hs, p);
-        else hipLaunchKernelGGL((k_seq_gemv<DT, ODT, 8, 4>), dim3((unsigned)((p.n + 15) / 16)), dim3(256), 0, hs, p);
+        if (p.m <= 2) hipLaunchKernelGGL((k_seq_gemv<DT, ODT, 2, 1, EPI>), dim3((unsigned)((p.n + 3) / 4)), dim3(256), 0, hs, p);
+        else if (p.m <= 4) hipLaunchKernelGGL((k_seq_gemv<DT, ODT, 4, 2, EPI>), dim3((unsigned)((p.n + 7) / 8)), dim3(256), 0, hs, p);
+        else hipLaunchKernelGGL((k_seq_gemv<DT, ODT, 8, 4, EPI>), dim3((unsigned)((p.n + 15) / 16)), dim3(256), 0, hs, p);
     } else {
-        launch_tiled<DT, ODT>(p, hs);
+        launch_tiled<DT, ODT, EPI>(p, hs);
     }
     return zl_launch_status();
 }
@@ -373,21 +388,32 @@ int launch(const GemmP& p, hipStream_t hs) {
 
 extern "C" int zls_version(void) { return 1; }
 
-extern "C" int zls_gemm_nt(const void* x, int64_t ldx, const void* w, void* y, int64_t ldy, int64_t m, int64_t n, int64_t k, int dtype,
-                           int out_dtype, zl_stream_t s) {
+extern "C" int zls_gemm_nt_act(const void* x, int64_t ldx, const void* w, const float* bias, int act, void* y, int64_t ldy, void* y2, int64_t ldy2,
+                               int64_t n2, int64_t m, int64_t n, int64_t k, int dtype, int out_dtype, zl_stream_t s) {
     ZL_CHECK_ARG(x && w && y && m > 0 && n > 0 && k > 0, ZL_EINVAL);
     ZL_CHECK_ARG(ldx >= k && ldy >= n && m < (1 << 30) && n < (1 << 30) && k < (1 << 30), ZL_ESHAPE);
     ZL_CHECK_ARG((m + 63) / 64 <= 65535, ZL_ELIMIT);
     ZL_CHECK_ARG(dtype == ZL_BF16 || dtype == ZL_F32, ZL_EDTYPE);
     ZL_CHECK_ARG(out_dtype == ZL_F32 || out_dtype == dtype, ZL_EDTYPE);
+    ZL_CHECK_ARG(act >= -1 && act <= 3 && (!y2 || (n2 > 0 && n2 <= n && ldy2 >= n2)), ZL_EINVAL);
     GemmP p = {};
     p.x = x; p.w = w; p.y = y; p.ldx = ldx; p.ldw = k; p.ldy = ldy; p.m = (int)m; p.n = (int)n; p.k = (int)k;
     p.x_rows = p.w_rows = nullptr; p.tiles = nullptr; p.w_stride = 0;
+    p.bias = bias; p.uact = act; p.y2 = y2; p.ldy2 = ldy2; p.n2 = y2 ? (int)n2 : 0;
     const int64_t unit = dtype == ZL_BF16 ? 8 : 4;
     p.vec = (k % unit == 0 && ldx % unit == 0 && ((uintptr_t)x & 15) == 0 && ((uintptr_t)w & 15) == 0) ? 1 : 0;
     hipStream_t hs = (hipStream_t)s;
+    if (bias || act >= 0 || y2) {
+        if (dtype == ZL_BF16) return out_dtype == ZL_F32 ? launch<ZL_BF16, ZL_F32, true>(p, hs) : launch<ZL_BF16, ZL_BF16, true>(p, hs);
+        return launch<ZL_F32, ZL_F32, true>(p, hs);
+    }
     if (dtype == ZL_BF16) return out_dtype == ZL_F32 ? launch<ZL_BF16, ZL_F32>(p, hs) : launch<ZL_BF16, ZL_BF16>(p, hs);
     return launch<ZL_F32, ZL_F32>(p, hs);
+}
+
+extern "C" int zls_gemm_nt(const void* x, int64_t ldx, const void* w, void* y, int64_t ldy, int64_t m, int64_t n, int64_t k, int dtype,
+                           int out_dtype, zl_stream_t s) {
+    return zls_gemm_nt_act(x, ldx, w, nullptr, -1, y, ldy, nullptr, 0, 0, m, n, k, dtype, out_dtype, s);
 }
 
 // the same product with GATHERED rows of x and / or w (x_rows / w_rows: device int32 row indices, NULL: the rows in order), always on the

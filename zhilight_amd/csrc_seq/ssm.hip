@@ -1,9 +1,8 @@
 // ssm.hip -- the state-space (Mamba-2) mixer's steps over a ragged step: causal short convolution + SiLU with a carried tail, the
 // selective recurrence with its fp32 state carried per sequence slot, the gated grouped RMS norm.
 //
-// k_conv_silu         a thread per (token, channel); taps before the portion come from the slot's tail (oldest row first)
-// k_conv_tail_update  after it: a thread per (sequence, channel) shifts the tail by the portion's length (rows in increasing order, each
-//                     read before it is overwritten)
+// k_conv_silu         a thread per (token, channel); taps before the portion come from the slot's tail (oldest row first), which moves on by
+//                     the portion's length in the same launch
 // k_ssm_scan          a workgroup per (sequence, head); the state in registers, tokens staged through LDS 16 at a time and walked in order;
 //                     dt, the decay and the state are fp32.  The same kernel runs linear attention with a scalar decay per head and token
 //                     (zls_decay_scan: x = v, B = k, C = q from columns of one projection, the decay and input scale given per token or
@@ -14,41 +13,35 @@
 namespace {
 
 // in_bias (nullable) is added to every INPUT of the convolution (the tail holds inputs with it; before a sequence's start the input is 0,
-// not the bias); act 0 leaves out the SiLU
+// not the bias); act 0 leaves out the SiLU; out_t (nullable): the result once more in the serving format.  The workgroups of a portion's
+// first token also do its tokens up to taps - 2 -- the only ones that look into the carried tail -- and, when those are done, move the
+// portion's last inputs into the tail (a thread owns its channels: rows in increasing order, each read before it is overwritten)
+template <int DT>
 __global__ __launch_bounds__(256) void k_conv_silu(const float* __restrict__ proj, int64_t ld, int col0, const float* __restrict__ w,
                                                    const float* __restrict__ bias, const float* __restrict__ in_bias, int act,
-                                                   const float* __restrict__ tail, int channels, int taps, const zls_batch_t b,
-                                                   float* __restrict__ out) {
+                                                   float* __restrict__ tail, int channels, int taps, const zls_batch_t b,
+                                                   float* __restrict__ out, void* __restrict__ out_t) {
     const int t = blockIdx.x;
     const int sq = b.tok_seq[t];
-    const int first = b.seq_start[sq];
-    const int i = t - first;                                           // index inside the portion
-    const float* tl = tail + (size_t)b.seq_slot[sq] * (taps - 1) * channels;
-    for (int c = blockIdx.y * 256 + threadIdx.x; c < channels; c += gridDim.y * 256) {
-        float a = bias ? bias[c] : 0.f;
-        const float ib = in_bias ? in_bias[c] : 0.f;
-        for (int k = 0; k < taps; ++k) {
-            const int back = taps - 1 - k;                             // the last column is the current token's
-            const int src = i - back;
-            const float u = src >= 0 ? proj[(size_t)(first + src) * ld + col0 + c] + ib
-                                     : tl[(size_t)(taps - 1 + src) * channels + c];     // src = -1 is the newest tail row
-            a = fmaf(w[(size_t)c * taps + k], u, a);
-        }
-        out[(size_t)t * channels + c] = act ? seq_silu(a) : a;
-    }
-}
-
-__global__ __launch_bounds__(256) void k_conv_tail_update(const float* __restrict__ proj, int64_t ld, int col0, const float* __restrict__ in_bias,
-                                                          float* __restrict__ tail, int channels, int taps, const zls_batch_t b) {
-    const int sq = blockIdx.x;
     const int first = b.seq_start[sq], count = b.seq_start[sq + 1] - first;
+    const int i0 = t - first;                                          // index inside the portion
+    if (i0 > 0 && i0 < taps - 1) return;
+    const int n = i0 == 0 ? max(1, min(count, taps - 1)) : 1;
     float* tl = tail + (size_t)b.seq_slot[sq] * (taps - 1) * channels;
     for (int c = blockIdx.y * 256 + threadIdx.x; c < channels; c += gridDim.y * 256) {
-        for (int j = 0; j < taps - 1; ++j) {                           // new row j = input at portion index count - (taps - 1) + j
-            const int src = count - (taps - 1) + j;
-            tl[(size_t)j * channels + c] = src >= 0 ? proj[(size_t)(first + src) * ld + col0 + c] + (in_bias ? in_bias[c] : 0.f)
-                                                    : tl[(size_t)(taps - 1 + src) * channels + c];   // an older row j + count > j
+        const float ib = in_bias ? in_bias[c] : 0.f;
+        auto input = [&](int src) {                                    // src = -1 is the newest tail row
+            return src >= 0 ? proj[(size_t)(first + src) * ld + col0 + c] + ib : tl[(size_t)(taps - 1 + src) * channels + c];
+        };
+        for (int i = i0; i < i0 + n; ++i) {
+            float a = bias ? bias[c] : 0.f;
+            for (int k = 0; k < taps; ++k) a = fmaf(w[(size_t)c * taps + k], input(i - (taps - 1 - k)), a);      // (the last column: the current token's)
+            a = act ? seq_silu(a) : a;
+            out[(size_t)(first + i) * channels + c] = a;
+            if (out_t) SeqT<DT>::st(out_t, (size_t)(first + i) * channels + c, a);
         }
+        if (i0 == 0)
+            for (int j = 0; j < taps - 1; ++j) tl[(size_t)j * channels + c] = input(count - (taps - 1) + j);     // (an older row j + count > j, or an input)
     }
 }
 
@@ -285,35 +278,20 @@ __global__ __launch_bounds__(256) void k_gated_group_norm(const float* __restric
 }  // namespace
 
 extern "C" int zls_short_conv(const float* proj, int64_t ld, int64_t col0, const float* w, const float* bias, const float* in_bias, int act,
-                              const float* tail, int64_t channels, int64_t taps, const zls_batch_t* b, float* out, zl_stream_t s) {
+                              float* tail, int64_t channels, int64_t taps, const zls_batch_t* b, float* out, void* out_t, int dtype, zl_stream_t s) {
     ZL_CHECK_ARG(proj && w && out && seq_batch_ok(b) && channels > 0 && taps > 0 && (tail || taps == 1), ZL_EINVAL);
     ZL_CHECK_ARG(col0 >= 0 && col0 + channels <= ld, ZL_ESHAPE);
     const unsigned gy = (unsigned)((channels + 255) / 256 > 64 ? 64 : (channels + 255) / 256);
-    hipLaunchKernelGGL(k_conv_silu, dim3(b->n_tok, gy), dim3(256), 0, (hipStream_t)s, proj, ld, (int)col0, w, bias, in_bias, act ? 1 : 0, tail,
-                       (int)channels, (int)taps, *b, out);
+#define CALL(DT) hipLaunchKernelGGL((k_conv_silu<DT>), dim3(b->n_tok, gy), dim3(256), 0, (hipStream_t)s, proj, ld, (int)col0, w, bias, in_bias, \
+                                    act ? 1 : 0, tail, (int)channels, (int)taps, *b, out, out_t);
+    ZLS_DISPATCH(dtype, CALL)
+#undef CALL
     return zl_launch_status();
 }
 
-extern "C" int zls_conv_silu(const float* proj, int64_t ld, int64_t col0, const float* w, const float* bias, const float* tail, int64_t channels,
+extern "C" int zls_conv_silu(const float* proj, int64_t ld, int64_t col0, const float* w, const float* bias, float* tail, int64_t channels,
                              int64_t taps, const zls_batch_t* b, float* out, zl_stream_t s) {
-    return zls_short_conv(proj, ld, col0, w, bias, nullptr, 1, tail, channels, taps, b, out, s);
-}
-
-extern "C" int zls_short_conv_tail(const float* proj, int64_t ld, int64_t col0, const float* in_bias, float* tail, int64_t channels, int64_t taps,
-                                   const zls_batch_t* b, zl_stream_t s) {
-    ZL_CHECK_ARG(proj && seq_batch_ok(b) && channels > 0 && taps > 0, ZL_EINVAL);
-    ZL_CHECK_ARG(col0 >= 0 && col0 + channels <= ld, ZL_ESHAPE);
-    if (taps == 1) return ZL_OK;
-    ZL_CHECK_ARG(tail, ZL_EINVAL);
-    const unsigned gy = (unsigned)((channels + 255) / 256 > 64 ? 64 : (channels + 255) / 256);
-    hipLaunchKernelGGL(k_conv_tail_update, dim3(b->n_seq, gy), dim3(256), 0, (hipStream_t)s, proj, ld, (int)col0, in_bias, tail, (int)channels,
-                       (int)taps, *b);
-    return zl_launch_status();
-}
-
-extern "C" int zls_conv_tail_update(const float* proj, int64_t ld, int64_t col0, float* tail, int64_t channels, int64_t taps, const zls_batch_t* b,
-                                    zl_stream_t s) {
-    return zls_short_conv_tail(proj, ld, col0, nullptr, tail, channels, taps, b, s);
+    return zls_short_conv(proj, ld, col0, w, bias, nullptr, 1, tail, channels, taps, b, out, nullptr, ZL_F32, s);
 }
 
 extern "C" int64_t zls_ssm_scan_workspace_bytes(int64_t n_seq, int64_t max_count, int64_t seg_len, int64_t heads, int64_t vdim, int64_t n_state) {

@@ -27,9 +27,11 @@ constexpr int kChunk = 128;         // the largest page k_window_attention walks
 constexpr int kMaxV = 8;            // output coordinates per thread: (all_kv ? kv_heads : 1) * vdim <= 256 * kMaxV
 
 // one head of `size` coordinates in the lanes' registers (coordinate i in lane i % 64, register i / 64): rotate the first n_rot (pairs
-// i, i + n_rot / 2; interleaved: pairs 2i, 2i + 1) by pos * freq[i], optionally divide by the root mean square; the result stays in v[]
+// i, i + n_rot / 2; interleaved: pairs 2i, 2i + 1) by pos * freq[i], optionally divide by the root mean square; the result stays in v[].
+// pre / pre_w: a factor and a weight per coordinate that the numbers get before anything else
 __device__ __forceinline__ void rope_head(float* v, const float* src, int size, int n_rot, const float* __restrict__ freq, float pos, bool norm,
-                                          float eps, int lane, bool interleaved = false, const float* __restrict__ w = nullptr) {
+                                          float eps, int lane, bool interleaved = false, const float* __restrict__ w = nullptr, float pre = 1.0f,
+                                          const float* __restrict__ pre_w = nullptr) {
     const int half = n_rot >> 1;
     float ss = 0.f;
 #pragma unroll
@@ -37,10 +39,11 @@ __device__ __forceinline__ void rope_head(float* v, const float* src, int size, 
         const int i = lane + 64 * r;
         float o = 0.f;
         if (i < size) {
-            o = src[i];
+            o = pre_w ? src[i] * pre * pre_w[i] : src[i] * pre;
             if (i < n_rot) {
                 const bool lo = interleaved ? (i & 1) == 0 : i < half;
-                const float other = src[interleaved ? (i ^ 1) : (lo ? i + half : i - half)];
+                const int oi = interleaved ? (i ^ 1) : (lo ? i + half : i - half);
+                const float other = pre_w ? src[oi] * pre * pre_w[oi] : src[oi] * pre;
                 float sn, cs;
                 seq_sincos(pos * freq[interleaved ? (i >> 1) : (lo ? i : i - half)], &sn, &cs);
                 o = lo ? o * cs - other * sn : o * cs + other * sn;
@@ -65,6 +68,7 @@ struct RopeP {
     int interleaved;
     const float* vmix_src; int64_t vmix_ld; int vmix_col0; float vmix_lambda;     // values <- (1 - lambda) values + lambda vmix_src[t][col0 ..]
     const float* q_w; const float* k_w;             // nullable (dim): weights of the query / key norm, shared by the heads
+    zls_head_prep_t prep;                           // norms over whole rows, query temperature, further heads (all zero: none)
 };
 
 template <int DT>
@@ -77,17 +81,40 @@ __global__ __launch_bounds__(256) void k_rope_norm_store(const RopeP p, const zl
     const size_t cpage = (size_t)b.page_table[(size_t)sq * b.max_pages + posi / b.page_size];
     const size_t crow = cpage * b.page_size + posi % b.page_size;
     const int n_kv = p.k_cache ? p.kv_heads : 0;
+    float fq = 1.0f, fk = 1.0f, temp = 1.0f;
+    if (p.prep.whole_norm) {                                             // one root mean square over all query heads, one over all key heads
+        __shared__ float red[16];
+        const int nq = p.heads * p.dim, nk = n_kv * p.dim;
+        float sq_ = 0.f, sk_ = 0.f;
+        for (int i = threadIdx.x; i < nq; i += 256) { const float u = row[p.q_col0 + i]; sq_ = fmaf(u, u, sq_); }
+        for (int i = threadIdx.x; i < nk; i += 256) { const float u = row[p.k_col0 + i]; sk_ = fmaf(u, u, sk_); }
+        fq = 1.0f / sqrtf(zl_block_sum(sq_, red) / (float)nq + p.eps);   // (its barriers: every wave has read the row before one writes it)
+        if (nk) fk = 1.0f / sqrtf(zl_block_sum(sk_, red) / (float)nk + p.eps);
+    }
+    if (p.prep.temp_every > 0) temp = 1.0f + p.prep.temp_coef * logf((float)((posi + 1) / p.prep.temp_every + 1));
     float v[kMaxE];
-    for (int h = wave; h < p.heads + 2 * n_kv; h += 4) {                 // (a wave owns its heads: no two waves touch the same numbers)
-        if (h < p.heads) {
+    for (int h = wave; h < p.heads + 2 * n_kv + p.prep.x_heads; h += 4) {          // (a wave owns its heads: no two waves touch the same numbers)
+        if (h >= p.heads + 2 * n_kv) {
+            float* x = row + p.prep.x_col0 + (h - p.heads - 2 * n_kv) * p.prep.x_dim;
+            rope_head(v, x, p.prep.x_dim, p.prep.x_rot, p.prep.x_freq, pos, false, 0.f, lane);
+#pragma unroll
+            for (int r = 0; r < kMaxE; ++r)
+                if (lane + 64 * r < p.prep.x_rot) x[lane + 64 * r] = v[r];
+        } else if (h < p.heads) {
             float* q = row + p.q_col0 + h * p.dim;
-            rope_head(v, q, p.dim, p.rot_dims, p.qk_freq, pos, p.qk_norm != 0, p.eps, lane, p.interleaved != 0, p.q_w);
+            rope_head(v, q, p.dim, p.rot_dims, p.qk_freq, pos, p.qk_norm != 0, p.eps, lane, p.interleaved != 0, p.q_w, fq,
+                      p.prep.q_w ? p.prep.q_w + h * p.dim : nullptr);
+            if (p.prep.temp_every > 0) {
+#pragma unroll
+                for (int r = 0; r < kMaxE; ++r) v[r] *= temp;
+            }
 #pragma unroll
             for (int r = 0; r < kMaxE; ++r)
                 if (lane + 64 * r < p.dim) q[lane + 64 * r] = v[r];
         } else if (h < p.heads + n_kv) {
             const int c = h - p.heads;
-            rope_head(v, row + p.k_col0 + c * p.dim, p.dim, p.rot_dims, p.qk_freq, pos, p.qk_norm != 0, p.eps, lane, p.interleaved != 0, p.k_w);
+            rope_head(v, row + p.k_col0 + c * p.dim, p.dim, p.rot_dims, p.qk_freq, pos, p.qk_norm != 0, p.eps, lane, p.interleaved != 0, p.k_w, fk,
+                      p.prep.k_w ? p.prep.k_w + c * p.dim : nullptr);
 #pragma unroll
             for (int r = 0; r < kMaxE; ++r)
                 if (lane + 64 * r < p.dim) SeqT<DT>::st(p.k_cache, (crow * p.kv_heads + c) * p.dim + lane + 64 * r, v[r]);
@@ -143,12 +170,14 @@ struct AttnP {
     const float* offset;                   // (heads) sigmoid weights: w = sigmoid(score + offset[g])
     int chunk;                             // > 0: a query only sees the keys of its own chunk of `chunk` positions, counted from position 0
     int sigmoid;                           // weights are sigmoids, each key on its own: no maximum, no normaliser (ml = (0, 1) for a split with keys)
+    const float* slope;                    // (heads) slope[g] * (p - j) is taken off the (capped) score
 };
 
 // the score of the general form from the scaled product
 __device__ __forceinline__ float form_score(const AttnP& p, float s, int g, int dist) {
     if (p.softcap > 0.f) s = p.softcap * tanhf(s / p.softcap);
     if (p.bias) s += p.bias[(size_t)g * p.bias_rows + min(dist, p.bias_rows - 1)];
+    if (p.slope) s = fmaf(-p.slope[g], (float)dist, s);
     return s;
 }
 
@@ -299,11 +328,12 @@ __device__ __forceinline__ float fast_sigmoid(float x) {
 __device__ __forceinline__ float fast_tanh(float x) { return 2.0f * fast_sigmoid(2.0f * x) - 1.0f; }
 
 template <int KS, int FORM>             // 32-coordinate steps of the head size: dim <= 32 KS; FORM 1: the general score form of AttnP with a
-                                        // softmax, 2: with sigmoid weights (no maximum, no correction of the sums, no normaliser)
+                                        // softmax, 2: with sigmoid weights (no maximum, no correction of the sums, no normaliser),
+                                        // 3: a softmax whose only addition is the linear distance bias (slope)
 __global__ __launch_bounds__(256) void k_window_attention_mfma(const AttnP p, const zls_batch_t b) {
     __shared__ uint4 pfrag[2][4][2][2][64];                              // [buffer][query block][key half][hi, lo][lane]
     __shared__ float corr_s[2][64], l_s[64], m_s[64];
-    __shared__ float bias_s[FORM ? kBiasLds : 1];
+    __shared__ float bias_s[(FORM == 1 || FORM == 2) ? kBiasLds : 1];
     const int tile = blockIdx.x, g = blockIdx.y, part = blockIdx.z;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, nrow = lane & 15, kq = lane >> 4;
     const int t0 = p.tiles[3 * tile], rows = p.tiles[3 * tile + 1], sq = p.tiles[3 * tile + 2];
@@ -322,7 +352,7 @@ __global__ __launch_bounds__(256) void k_window_attention_mfma(const AttnP p, co
     const int chunk0 = (FORM && p.chunk > 0) ? pq / p.chunk * p.chunk : 0;          // the first position of the query's chunk
     const float off = (FORM && p.offset) ? p.offset[g] : 0.f;
     const float inv_cap = (FORM && p.softcap > 0.f) ? 1.0f / p.softcap : 0.f;
-    const bool bias_lds = FORM && p.bias && p.bias_rows <= kBiasLds;     // (uniform: the whole row of the head sits in LDS)
+    const bool bias_lds = (FORM == 1 || FORM == 2) && p.bias && p.bias_rows <= kBiasLds;     // (uniform: the whole row of the head sits in LDS)
     // Sigmoid weights (FORM 2) in as few instructions per score as the form allows.  With r = 1 / (1 + 2^(k1 s)), k1 = -2 log2(e) / cap,
     // the capped score is 2 cap r - cap, so the weight is 1 / (1 + 2^z) with z = A r + b[distance]: A = -2 cap log2(e) and
     // b = -log2(e) (bias + offset - cap), which is what the LDS row holds here; without a cap r = s and A = -log2(e).
@@ -335,7 +365,8 @@ __global__ __launch_bounds__(256) void k_window_attention_mfma(const AttnP p, co
     const bool fast_vis = FORM == 2 && p.keep_first == 0;
     const int pq_eff = qok ? pq : -(1 << 30);
     const unsigned dmax = qok ? (unsigned)min(pq - chunk0, p.window > 0 ? p.window - 1 : pq) : 0u;
-    if (FORM && p.bias) {
+    const float slope = (FORM && p.slope) ? p.slope[g] : 0.f;
+    if ((FORM == 1 || FORM == 2) && p.bias) {
         for (int i = tid; i < min(p.bias_rows, kBiasLds); i += 256) {
             const float bv = p.bias[(size_t)g * p.bias_rows + i];
             bias_s[i] = FORM == 2 ? fmaf(-kL2e, bv, sg_c0) : bv;
@@ -422,8 +453,9 @@ __global__ __launch_bounds__(256) void k_window_attention_mfma(const AttnP p, co
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int j = pg * 64 + 16 * kb + 4 * kq + r;
-                vis[kb][r] = qok && j <= pq && (p.window <= 0 || pq - j < p.window || j < p.keep_first) && (!FORM || j >= chunk0);
-                if (FORM && vis[kb][r]) {
+                vis[kb][r] = qok && j <= pq && (p.window <= 0 || pq - j < p.window || j < p.keep_first) && (FORM == 0 || FORM == 3 || j >= chunk0);
+                if (FORM == 3) st[kb][r] = fmaf(slope, (float)(j - pq), st[kb][r]);      // (the distance is an exact fp32 number)
+                if (FORM == 1 && vis[kb][r]) {
                     float sv = st[kb][r];
                     if (p.softcap > 0.f) sv = p.softcap * fast_tanh(sv * inv_cap);
                     if (bias_lds) sv += bias_s[min(pq - j, p.bias_rows - 1)];
@@ -431,6 +463,7 @@ __global__ __launch_bounds__(256) void k_window_attention_mfma(const AttnP p, co
                         const int bi = min(pq - j, p.bias_rows - 1);
                         sv += bi < kBiasLds ? bias_s[bi] : p.bias[(size_t)g * p.bias_rows + bi];
                     }
+                    if (p.slope) sv = fmaf(slope, (float)(j - pq), sv);
                     st[kb][r] = sv;
                 }
                 if (FORM != 2 && vis[kb][r]) cm = fmaxf(cm, st[kb][r]);
@@ -652,15 +685,22 @@ __global__ __launch_bounds__(256) void k_head_mix_gate(const MixP p, const zls_b
 extern "C" int zls_rope_norm_store(float* proj, int64_t ld, int64_t q_col0, int64_t k_col0, int64_t v_col0, int64_t heads, int64_t kv_heads,
                                    int64_t dim, int64_t vdim, const float* qk_freq, int64_t rot_dims, const float* v_freq, float eps, int qk_norm,
                                    int interleaved, const float* vmix_src, int64_t vmix_ld, int64_t vmix_col0, float vmix_lambda,
-                                   const float* q_norm_w, const float* k_norm_w, const zls_batch_t* b, void* k_cache, void* v_cache, int dtype,
-                                   zl_stream_t s) {
+                                   const float* q_norm_w, const float* k_norm_w, const zls_head_prep_t* prep, const zls_batch_t* b, void* k_cache,
+                                   void* v_cache, int dtype, zl_stream_t s) {
     ZL_CHECK_ARG(proj && seq_batch_ok(b) && b->page_table && b->page_size > 0 && heads > 0 && kv_heads > 0 && dim > 0 && vdim > 0, ZL_EINVAL);
     ZL_CHECK_ARG((k_cache == nullptr) == (v_cache == nullptr), ZL_EINVAL);
     ZL_CHECK_ARG(rot_dims >= 0 && rot_dims <= dim && rot_dims % 2 == 0 && (rot_dims == 0 || qk_freq) && (!v_freq || vdim % 2 == 0), ZL_ESHAPE);
     ZL_CHECK_ARG(dim <= 64 * kMaxE && vdim <= 64 * kMaxE, ZL_ELIMIT);
     ZL_CHECK_ARG(q_col0 >= 0 && q_col0 + heads * dim <= ld, ZL_ESHAPE);
     ZL_CHECK_ARG(!k_cache || (k_col0 >= 0 && k_col0 + kv_heads * dim <= ld && v_col0 >= 0 && v_col0 + kv_heads * vdim <= ld), ZL_ESHAPE);
-    RopeP p;
+    RopeP p = {};
+    if (prep) {
+        ZL_CHECK_ARG(!(prep->whole_norm && qk_norm) && prep->temp_every >= 0, ZL_EINVAL);
+        ZL_CHECK_ARG(prep->x_heads >= 0 && (prep->x_heads == 0 || (prep->x_dim > 0 && prep->x_dim <= 64 * kMaxE && prep->x_rot >= 0 && prep->x_rot % 2 == 0 &&
+                     prep->x_rot <= prep->x_dim && (prep->x_rot == 0 || prep->x_freq) && prep->x_col0 >= 0 &&
+                     prep->x_col0 + (int64_t)prep->x_heads * prep->x_dim <= ld)), ZL_ESHAPE);
+        p.prep = *prep;
+    }
     p.proj = proj; p.ld = ld; p.q_col0 = (int)q_col0; p.k_col0 = (int)k_col0; p.v_col0 = (int)v_col0; p.heads = (int)heads;
     p.kv_heads = (int)kv_heads; p.dim = (int)dim; p.vdim = (int)vdim; p.rot_dims = (int)rot_dims; p.qk_norm = qk_norm; p.qk_freq = qk_freq;
     p.v_freq = v_freq; p.eps = eps; p.k_cache = k_cache; p.v_cache = v_cache;
@@ -679,7 +719,8 @@ static int set_form(AttnP& p, const zls_score_form_t* f) {
     ZL_CHECK_ARG((!f->bias || f->bias_rows > 0) && f->chunk >= 0 && f->chunk < (1 << 30), ZL_ESHAPE);
     ZL_CHECK_ARG(!(f->chunk > 0 && p.keep_first > 0), ZL_ESHAPE);        // (kept first keys belong to a sliding window, not to chunks)
     p.head_scale = f->head_scale; p.softcap = f->softcap; p.bias = f->bias; p.bias_rows = f->bias_rows; p.offset = f->offset;
-    p.chunk = f->chunk; p.sigmoid = f->sigmoid ? 1 : 0;
+    ZL_CHECK_ARG(!(f->slope && f->sigmoid), ZL_ESHAPE);                  // (sigmoid weights take their distance bias as a table)
+    p.chunk = f->chunk; p.sigmoid = f->sigmoid ? 1 : 0; p.slope = f->slope;
     return ZL_OK;
 }
 
@@ -730,8 +771,10 @@ extern "C" int zls_window_attention_prompt(const float* q, int64_t ldq, int64_t 
     const dim3 grid((unsigned)n_tiles, (unsigned)heads, (unsigned)parts);
     hipStream_t hs = (hipStream_t)s;
     const int ks = (int)((dim + 31) / 32);
+    const bool only_slope = form && form->slope && !form->head_scale && !(form->softcap > 0.f) && !form->bias && form->chunk == 0;
 #define PROMPT(KS)                                                                                      \
     if (form && form->sigmoid) hipLaunchKernelGGL((k_window_attention_mfma<KS, 2>), grid, dim3(256), 0, hs, p, *b); \
+    else if (only_slope) hipLaunchKernelGGL((k_window_attention_mfma<KS, 3>), grid, dim3(256), 0, hs, p, *b); \
     else if (form) hipLaunchKernelGGL((k_window_attention_mfma<KS, 1>), grid, dim3(256), 0, hs, p, *b); \
     else hipLaunchKernelGGL((k_window_attention_mfma<KS, 0>), grid, dim3(256), 0, hs, p, *b)
     if (ks <= 1) { PROMPT(1); }

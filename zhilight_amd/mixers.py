@@ -6,6 +6,7 @@ between steps it registers with the CacheManager in `bind`: per-token rows as a 
 All per-sequence arithmetic that must not lose bits (norms, softmax, the recurrence, its state) is fp32 inside the kernels in both serving
 formats; matrices are in the serving format, small vectors fp32.
 """
+import copy
 import math
 
 import torch
@@ -30,6 +31,16 @@ def _vec(get, name, n, device):
 
 def _rand(gen, shape, std, dtype, device):
     return (torch.randn(shape, generator=gen, device=device, dtype=torch.float32) * std).to(dtype)
+
+
+def replica(mixer, name):
+    """The same mixer -- the same weight tensors -- under another name: once bound it keeps a cache or state of its own.  For layers that run
+    several times over a sequence with shared weights."""
+    m = copy.copy(mixer)
+    m.name = name
+    for part in getattr(mixer, "parts", ()):
+        setattr(m, part, replica(getattr(mixer, part), name + "." + part))
+    return m
 
 
 class SideRows:
@@ -270,6 +281,12 @@ def distance_bias_table(rel, far, longest, device):
     return rel.to(torch.float32)[row.to(rel.device)].t().contiguous().to(device)
 
 
+def linear_slopes(heads, device):
+    """2^(-8 (h + 1) / heads) for h = 0 .. heads - 1, worked out in float64 and rounded once to fp32"""
+    h = torch.arange(heads, dtype=torch.float64)
+    return torch.exp2(-8.0 * (h + 1.0) / heads).to(torch.float32).to(device)
+
+
 class WindowAttention(SideRows):
     """Softmax attention with grouped key / value heads over a paged cache: rotary positions on the first `rot_dims` coordinates of every
     query and key head (pairs i, i + rot_dims / 2; every frequency divided by `rot_scaling`), queries and keys divided by their root mean
@@ -291,14 +308,17 @@ class WindowAttention(SideRows):
         added after the cap (rel_far > 0; tensor `rel` (rows, heads), see distance_bias_table),
       * queries that only see the keys of their own chunk of `chunk` positions, chunks counted from position 0 of the sequence,
       * weights that are no softmax: weights="sigmoid" gives every visible key sigmoid(score + offset_h) (tensor `pb` (heads)), not
-        normalised over the keys.
+        normalised over the keys,
+      * ONE norm over all query heads and one over all key heads, right after the projection (whole_norm; tensors q.norm (heads*dim), k.norm
+        (kv_heads*dim)), queries multiplied by 1 + coef ln(floor((p + 1) / every) + 1) at position p (q_temp = (coef, every)),
+      * a linear distance bias: slope_h (p - j) is taken off the score, slope_h = 2^(-8 (h + 1) / heads) (slope_bias).
     Tensors under `prefix`: q (heads*dim, width), k (kv_heads*dim, width), v (kv_heads*vdim, width), talk (heads, heads), g (heads*vdim, width),
     o (width, heads*vdim).  q | k | v | g are one product."""
 
     def __init__(self, name, width, heads, kv_heads, dim, vdim, scale, window, rot_dims, rot_base, rot_scaling, eps, qk_norm=True,
                  rotate_values=True, talk=True, gate=True, kv_source=None, rope_interleaved=False, bias=False, conv_taps=0, keep_first=0,
                  sink=False, v_mix=False, v_mix_source=None, norm_weight=False, head_scale=False, softcap=0.0, rel_far=0, chunk=0,
-                 weights="softmax"):
+                 weights="softmax", whole_norm=False, q_temp=None, slope_bias=False):
         if weights not in ("softmax", "sigmoid") or (weights == "sigmoid" and (sink or talk)) or (chunk and keep_first) or chunk < 0:
             raise ZLError("attention: sigmoid weights have no sink and no mixing; chunks keep no first keys")
         if norm_weight and not qk_norm:
@@ -306,6 +326,10 @@ class WindowAttention(SideRows):
         self.norm_weight, self.has_head_scale, self.softcap, self.rel_far, self.chunk = bool(norm_weight), bool(head_scale), float(softcap or 0.0), \
             int(rel_far or 0), int(chunk or 0)
         self.sigmoid = weights == "sigmoid"
+        if whole_norm and (qk_norm or kv_source is not None) or (slope_bias and self.sigmoid):
+            raise ZLError("attention: one norm over all heads excludes a norm per head and borrowed keys; sigmoid weights have no slopes")
+        self.whole_norm, self.q_temp, self.slope_bias = bool(whole_norm), (None if q_temp is None else (float(q_temp[0]), int(q_temp[1]))), bool(slope_bias)
+        self.slope = self.prep = self.proj_bias = None
         self.q_norm_w = self.k_norm_w = self.temp = self.rel = self.offset = self.form = None
         if heads % kv_heads or rot_dims % 2 or rot_dims > dim or (rotate_values and vdim % 2):
             raise ZLError("attention: heads must divide by kv_heads, rotated sizes must be even and fit the head")
@@ -338,13 +362,24 @@ class WindowAttention(SideRows):
         self.qk_freq = rotary_frequencies(self.rot_dims, self.rot_base, self.rot_scaling, device) if self.rot_dims else None
         self.v_freq = rotary_frequencies(self.vdim, self.rot_base, 1.0, device) if self.rotate_values else None
         self.form = None
-        if self.has_head_scale or self.softcap > 0 or self.rel is not None or self.chunk or self.sigmoid:
-            self.form = seqops.score_form(self.heads, self.temp, self.softcap, self.rel, self.offset, self.chunk, self.sigmoid)
+        if self.slope_bias:
+            self.slope = linear_slopes(self.heads, device)
+        if self.has_head_scale or self.softcap > 0 or self.rel is not None or self.chunk or self.sigmoid or self.slope is not None:
+            self.form = seqops.score_form(self.heads, self.temp, self.softcap, self.rel, self.offset, self.chunk, self.sigmoid, self.slope)
+        self.set_prep()
+
+    def set_prep(self, extra=None):
+        """what the cache-writing launch does besides rotation and norms per head; extra: see seqops.head_prep"""
+        self.prep = None
+        if self.whole_norm or self.q_temp or extra:
+            self.prep = seqops.head_prep(self.whole_norm, *((self.q_norm_w, self.k_norm_w) if self.whole_norm else (None, None)), self.q_temp, extra)
 
     def _load_form(self, get, prefix, device):
         d, H = self.dim, self.heads
         if self.norm_weight:
             self.q_norm_w, self.k_norm_w = _vec(get, prefix + "q.norm", d, device), _vec(get, prefix + "k.norm", d, device)
+        if self.whole_norm:
+            self.q_norm_w, self.k_norm_w = _vec(get, prefix + "q.norm", H * d, device), _vec(get, prefix + "k.norm", self.kv_heads * d, device)
         if self.has_head_scale:
             self.temp = _vec(get, prefix + "temp", H, device)
         if self.rel_far:
@@ -372,8 +407,7 @@ class WindowAttention(SideRows):
             self.in_bias = torch.cat([_vec(get, prefix + n + ".b", sizes[n], device) for n in names]).contiguous()
         if self.taps:
             self.conv_w = torch.cat([_mat(get, prefix + n + ".conv", (sizes[n], self.taps), torch.float32, device) for n in names]).contiguous()
-        elif self.has_bias:
-            self.conv_w = torch.ones((sum(sizes[n] for n in names), 1), device=device)       # (one tap of weight 1: the bias alone)
+        self._place_bias()
         self.sink = _vec(get, prefix + "sink", H, device) if self.has_sink else None
         if self.v_mix:
             self.vmix_lambda = float(_vec(get, prefix + "vmix", 1, device)[0])
@@ -391,13 +425,13 @@ class WindowAttention(SideRows):
             self.in_bias = 0.1 * torch.randn(C, generator=gen, device=device)
         if self.taps:
             self.conv_w = torch.randn(C, self.taps, generator=gen, device=device) * self.taps ** -0.5
-        elif self.has_bias:
-            self.conv_w = torch.ones((C, 1), device=device)
+        self._place_bias()
         self.sink = torch.zeros(H, device=device) if self.has_sink else None
         self.vmix_lambda = 0.5 if self.v_mix else 0.0
         d = self.dim
-        if self.norm_weight:
-            self.q_norm_w, self.k_norm_w = 1.0 + 0.1 * torch.randn(d, generator=gen, device=device), 1.0 + 0.1 * torch.randn(d, generator=gen, device=device)
+        if self.norm_weight or self.whole_norm:
+            nq, nk = (d, d) if self.norm_weight else (H * d, self.kv_heads * d)
+            self.q_norm_w, self.k_norm_w = (1.0 + 0.1 * torch.randn(n, generator=gen, device=device) for n in (nq, nk))
         if self.has_head_scale:
             self.temp = 1.0 + 0.1 * torch.randn(H, generator=gen, device=device)
         if self.rel_far:
@@ -407,6 +441,12 @@ class WindowAttention(SideRows):
             self.offset = -2.0 + 0.1 * torch.randn(H, generator=gen, device=device)
         self._tables(device)
         return self
+
+    def _place_bias(self):
+        """biases without a convolution join the product itself (its epilogue; the gate's columns get zeros)"""
+        if self.has_bias and not self.taps:
+            self.proj_bias = torch.zeros(self._cols()[3], device=self.in_bias.device)
+            self.proj_bias[:self.in_bias.numel()] = self.in_bias
 
     def bind(self, cache, dtype):
         if self.kv_source is not None:                      # (the lender is an earlier layer: it is bound already)
@@ -421,56 +461,76 @@ class WindowAttention(SideRows):
         return sum(t.numel() * t.element_size() for t in (self.w_in, self.w_o))
 
     def forward(self, h, batch):
+        bias = self.proj_bias
+        if bias is not None and self.side_col0 is not None and bias.numel() != self.w_in.shape[0]:
+            bias = self.proj_bias = torch.cat([bias, torch.zeros(self.w_in.shape[0] - bias.numel(), device=bias.device)])
+        proj = seqops.gemm_nt(h, self.w_in, bias=bias)                            # fp32 [q | k | v | gate]
+        self.side = (proj, self.side_col0)
+        return seqops.gemm_nt(self.attend(proj, 0, batch, h.dtype), self.w_o)
+
+    def attend(self, proj, col0, batch, dtype):
+        """everything between the two products, from the fp32 columns [q | k | v | gate] of proj that start at col0 (biases are in them unless
+        a short convolution adds them); returns the output projection's input"""
         H, G, d, v = self.heads, self.kv_heads, self.dim, self.vdim
         k0, v0, g0, _ = self._cols()
         own = self.kv_source is None
-        proj = seqops.gemm_nt(h, self.w_in)                                       # fp32 [q | k | v | gate]
-        self.side = (proj, self.side_col0)
-        # biases and the short convolution give a second buffer [q | k | v] (the gate stays in proj); otherwise q is rotated inside proj
-        qkv = seqops.short_conv(proj, 0, self.conv_w, self.in_bias, self.tail, batch) if self.conv_w is not None else proj
+        # the short convolution gives a second buffer [q | k | v] (the gate stays in proj); otherwise q is rotated inside proj
+        qkv, c0 = (seqops.short_conv(proj, col0, self.conv_w, self.in_bias, self.tail, batch), 0) if self.conv_w is not None else (proj, col0)
         blend = None
         if self.v_mix and self.v_mix_source is not None:
             src, col = self.v_mix_source.last_values
             blend = (src, col, self.vmix_lambda)
-        self.last_values = (qkv, v0) if self.v_mix else None                      # (this step's values before blending, for a later layer)
-        seqops.rope_norm_store(qkv, 0, k0, v0, H, G, d, v, self.qk_freq, self.rot_dims, self.v_freq, self.eps, self.qk_norm, batch,
+        self.last_values = (qkv, c0 + v0) if self.v_mix else None                 # (this step's values before blending, for a later layer)
+        seqops.rope_norm_store(qkv, c0, c0 + k0, c0 + v0, H, G, d, v, self.qk_freq, self.rot_dims, self.v_freq, self.eps, self.qk_norm, batch,
                                self.k_cache if own else None, self.v_cache if own else None, interleaved=self.interleaved, vmix=blend,
-                               q_norm_w=self.q_norm_w, k_norm_w=self.k_norm_w)
-        acc, ml, n_splits = seqops.window_attention(qkv, 0, self.k_cache, self.v_cache, batch, self.scale, self.window, H, G, d, v,
+                               q_norm_w=self.q_norm_w if self.norm_weight else None, k_norm_w=self.k_norm_w if self.norm_weight else None,
+                               prep=self.prep)
+        acc, ml, n_splits = seqops.window_attention(qkv, c0, self.k_cache, self.v_cache, batch, self.scale, self.window, H, G, d, v,
                                                     all_kv=self.has_talk, mfma=self.prompt_kernel, n_splits=self.n_splits,
                                                     keep_first=self.keep_first, form=self.form)
-        a = seqops.head_mix_gate(acc, ml, n_splits, self.talk, self.v_freq, proj if self.has_gate else None, g0, batch, H, G, v, h.dtype,
-                                 sink=self.sink, plain_sum=self.sigmoid)
-        return seqops.gemm_nt(a, self.w_o)
+        return seqops.head_mix_gate(acc, ml, n_splits, self.talk, self.v_freq, proj if self.has_gate else None, col0 + g0, batch, H, G, v, dtype,
+                                    sink=self.sink, plain_sum=self.sigmoid)
 
 
 class DecayLinearAttention:
     """Linear attention with a fixed decay per head: q, k, v = act(projections); S_t = decay_h S_{t-1} + k_t v_t^T, o_t = S_t^T q_t per head,
-    the state fp32 per sequence; then the RMS norm over all heads together with a weight, the sigmoid gate, the output projection.
+    the state fp32 per sequence; then an RMS norm over `norm_groups` equal parts of the heads' outputs (1: all heads together, heads: each
+    head alone) with an optional weight, a gate -- sigmoid or silu of a projection (gate_act) --, the output projection.  Optionally (a
+    retention layer) q and k are rotated by their position over the first rot_dims coordinates of every head (pairs i, i + rot_dims / 2,
+    angle p * rot_base^(-2i / rot_dims)) and the keys multiplied by key_scale (the recurrence is linear in k: applied to o, before its norm).
     Tensors under `prefix`: q, k (heads*dim, width), v, g (heads*vdim, width), norm (heads*vdim), o (width, heads*vdim)."""
 
-    def __init__(self, name, width, heads, dim, vdim, decay, eps, act="silu", norm_groups=1):
+    def __init__(self, name, width, heads, dim, vdim, decay, eps, act="silu", norm_groups=1, norm_weight=True, gate_act="sigmoid", rot_dims=0,
+                 rot_base=10000.0, key_scale=1.0):
         if len(decay) != heads:
             raise ZLError("linear attention: one decay per head")
+        if rot_dims % 2 or not 0 <= rot_dims <= dim or (rot_dims and act is not None):
+            raise ZLError("linear attention: the rotated part is even and fits the head; rotated queries and keys have no activation")
         self.name, self.width, self.heads, self.dim, self.vdim = name, width, heads, dim, vdim
         self.decay_values, self.eps, self.act, self.norm_groups = [float(x) for x in decay], float(eps), act, norm_groups
+        self.has_norm_weight, self.gate_act, self.key_scale = bool(norm_weight), gate_act, float(key_scale)
+        self.rot_dims, self.rot_base = int(rot_dims), float(rot_base)
         self.scan_segment = None
+
+    def _constants(self, device):
+        self.decay = torch.tensor(self.decay_values, dtype=torch.float64).to(torch.float32).to(device)
+        self.freq = rotary_frequencies(self.rot_dims, self.rot_base, 1.0, device) if self.rot_dims else None
 
     def load(self, get, prefix, dtype, device):
         H, d, v, W = self.heads, self.dim, self.vdim, self.width
         self.w_in = torch.cat([_mat(get, prefix + "q", (H * d, W), dtype, device), _mat(get, prefix + "k", (H * d, W), dtype, device),
                                _mat(get, prefix + "v", (H * v, W), dtype, device), _mat(get, prefix + "g", (H * v, W), dtype, device)], dim=0).contiguous()
-        self.norm_w = _vec(get, prefix + "norm", H * v, device)
+        self.norm_w = _vec(get, prefix + "norm", H * v, device) if self.has_norm_weight else None
         self.w_o = _mat(get, prefix + "o", (W, H * v), dtype, device)
-        self.decay = torch.tensor(self.decay_values, dtype=torch.float64).to(torch.float32).to(device)
+        self._constants(device)
         return self
 
     def init_random(self, gen, dtype, device):
         H, d, v, W = self.heads, self.dim, self.vdim, self.width
         self.w_in = _rand(gen, (2 * H * d + 2 * H * v, W), W ** -0.5, dtype, device)
-        self.norm_w = torch.ones(H * v, device=device)
+        self.norm_w = torch.ones(H * v, device=device) if self.has_norm_weight else None
         self.w_o = _rand(gen, (W, H * v), (H * v) ** -0.5, dtype, device)
-        self.decay = torch.tensor(self.decay_values, dtype=torch.float32, device=device)
+        self._constants(device)
         return self
 
     def bind(self, cache, dtype):
@@ -479,13 +539,139 @@ class DecayLinearAttention:
     def weight_bytes(self):
         return sum(t.numel() * t.element_size() for t in (self.w_in, self.w_o))
 
+    def rotated(self, col0):
+        """the queries and keys behind col0 as heads to rotate in place (seqops.head_prep's `extra`); None without a rotation"""
+        return (col0, 2 * self.heads, self.dim, self.rot_dims, self.freq) if self.rot_dims else None
+
     def forward(self, h, batch):
-        H, d, v = self.heads, self.dim, self.vdim
         proj = seqops.gemm_nt(h, self.w_in)                                       # fp32 [q | k | v | gate]
-        y = seqops.decay_scan(proj, 0, H * d, 2 * H * d, self.act == "silu", self.decay, None, None, False, self.state, H, d, v, batch,
+        if self.rot_dims:                                                         # (queries and keys alike: 2 heads groups of one launch)
+            seqops.rope_norm_store(proj, 0, 0, 0, 2 * self.heads, 1, self.dim, 1, self.freq, self.rot_dims, None, self.eps, False, batch, None, None)
+        return seqops.gemm_nt(self.attend(proj, 0, batch, h.dtype), self.w_o)
+
+    def attend(self, proj, col0, batch, dtype):
+        """everything between the two products but the rotation, from the fp32 columns [q | k | v | gate] of proj that start at col0"""
+        H, d, v = self.heads, self.dim, self.vdim
+        y = seqops.decay_scan(proj, col0, col0 + H * d, col0 + 2 * H * d, self.act == "silu", self.decay, None, None, False, self.state, H, d, v, batch,
                               seg_len=self.scan_segment)
-        a = seqops.linear_attn_finish(y, False, 1.0, None, 0.0, H, v, self.norm_groups, self.norm_w, self.eps, proj, 2 * H * d + H * v, h.dtype)
-        return seqops.gemm_nt(a, self.w_o)
+        return seqops.linear_attn_finish(y, False, self.key_scale, None, 0.0, H, v, self.norm_groups, self.norm_w, self.eps, proj,
+                                         col0 + 2 * H * d + H * v, dtype, gate_act=self.gate_act)
+
+
+class ParallelMixers:
+    """Two mixers side by side on the same input: the first `left` (WindowAttention), the second `right` (DecayLinearAttention).  Their input
+    projections are ONE product [left | right]; one launch then norms, rotates and caches for both; their results join the residual with an
+    RMS norm over the model width each, as the branches (y, weight, coef) that seqops.add_branches sums.
+    Tensors under `prefix`: left.*, right.* (the mixers' own), left.out, right.out (width)."""
+    parts = ("left", "right")
+
+    def __init__(self, name, left, right, coef=0.5):
+        if left.width != right.width or left.conv_w is not None or left.taps or left.kv_source is not None:
+            raise ZLError("parallel mixers: one width; the left one projects its own keys and values and has no convolution")
+        self.name, self.width, self.left, self.right, self.coef = name, left.width, left, right, float(coef)
+
+    def _join(self):
+        left, right = self.left, self.right
+        self.w_in = torch.cat([left.w_in, right.w_in], dim=0).contiguous()
+        self.col = left.w_in.shape[0]                                             # (where the right mixer's columns start)
+        self.in_bias = None
+        if left.proj_bias is not None:
+            self.in_bias = torch.zeros(self.w_in.shape[0], device=self.w_in.device)
+            self.in_bias[:self.col] = left.proj_bias
+        left.w_in = right.w_in = None                                             # (the rows live in the joint matrix now)
+        left.set_prep(right.rotated(self.col))
+        return self
+
+    def load(self, get, prefix, dtype, device):
+        self.left.load(get, prefix + "left.", dtype, device)
+        self.right.load(get, prefix + "right.", dtype, device)
+        self.left_out, self.right_out = _vec(get, prefix + "left.out", self.width, device), _vec(get, prefix + "right.out", self.width, device)
+        return self._join()
+
+    def init_random(self, gen, dtype, device):
+        self.left.init_random(gen, dtype, device)
+        self.right.init_random(gen, dtype, device)
+        self.left_out, self.right_out = (1.0 + 0.1 * torch.randn(self.width, generator=gen, device=device) for _ in range(2))
+        return self._join()
+
+    def bind(self, cache, dtype):
+        self.left.bind(cache, dtype)
+        self.right.bind(cache, dtype)
+
+    def weight_bytes(self):
+        return sum(t.numel() * t.element_size() for t in (self.w_in, self.left.w_o, self.right.w_o))
+
+    def branches(self, h, batch):
+        proj = seqops.gemm_nt(h, self.w_in, bias=self.in_bias)                    # fp32 [left: q | k | v | right: q | k | v | gate]
+        a = self.left.attend(proj, 0, batch, h.dtype)                             # (its first launch also rotates the right mixer's q and k)
+        r = self.right.attend(proj, self.col, batch, h.dtype)
+        return [(seqops.gemm_nt(a, self.left.w_o), self.left_out, self.coef), (seqops.gemm_nt(r, self.right.w_o), self.right_out, self.coef)]
+
+
+class Mamba1Mixer:
+    """Selective state-space mixer with a decay per channel and state: [x | z] = W_in h; x through a causal short convolution (with bias) and
+    SiLU; [low | B | C] = W_x x; dt = softplus(W_dt low + bias) per channel; S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n with
+    A = -exp(A_log), y_c = sum_n S[c, n] C_n + D_c x_c; (y * silu(z)) to the output projection.  The state and the convolution's last inputs
+    are fp32 slot states.  The rows of `low` are padded to a multiple of 8 with zero rows (and W_dt with zero columns), so that the small
+    product reads aligned rows.
+    Tensors under `prefix`: in (2*inner, width), conv (inner, taps), conv.b (inner), x (rank + 2*n_state, inner), dt (inner, rank), dt.b
+    (inner), A_log (inner, n_state), D (inner), o (width, inner)."""
+
+    def __init__(self, name, width, inner, n_state, rank, taps):
+        if min(inner, n_state, rank, taps) < 1:
+            raise ZLError("mamba1: sizes must be positive")
+        self.name, self.width, self.inner, self.n_state, self.rank, self.taps = name, width, inner, n_state, rank, taps
+        self.low = (rank + 7) // 8 * 8
+        self.scan_segment = None          # tokens per segment of a long portion (None: seqops.SELECTIVE_SEGMENT; 0: never in segments)
+
+    def _pack(self, w_x, w_dt, a_log):
+        r, low = self.rank, self.low
+        pad = torch.zeros((low - r, self.inner), dtype=w_x.dtype, device=w_x.device)
+        self.w_x = torch.cat([w_x[:r], pad, w_x[r:]], dim=0).contiguous()
+        self.w_dt = torch.zeros((self.inner, low), dtype=w_dt.dtype, device=w_dt.device)
+        self.w_dt[:, :r] = w_dt
+        # the rates as exponents of two, (n_state, inner): exp(dt A) = 2^(dt a2)
+        self.a2 = (-torch.exp(a_log.double()) * math.log2(math.e)).to(torch.float32).t().contiguous()
+
+    def load(self, get, prefix, dtype, device):
+        C, N, R, W = self.inner, self.n_state, self.rank, self.width
+        self.w_in = _mat(get, prefix + "in", (2 * C, W), dtype, device)
+        self.conv_w = _mat(get, prefix + "conv", (C, self.taps), torch.float32, device)
+        self.conv_b, self.dt_bias, self.d = (_vec(get, prefix + n, C, device) for n in ("conv.b", "dt.b", "D"))
+        self._pack(_mat(get, prefix + "x", (R + 2 * N, C), dtype, device), _mat(get, prefix + "dt", (C, R), dtype, device),
+                   _mat(get, prefix + "A_log", (C, N), torch.float32, device))
+        self.w_o = _mat(get, prefix + "o", (W, C), dtype, device)
+        return self
+
+    def init_random(self, gen, dtype, device):
+        C, N, R, W = self.inner, self.n_state, self.rank, self.width
+        self.w_in = _rand(gen, (2 * C, W), W ** -0.5, dtype, device)
+        self.conv_w = _rand(gen, (C, self.taps), self.taps ** -0.5, torch.float32, device)
+        self.conv_b, self.d = torch.zeros(C, device=device), torch.ones(C, device=device)
+        self.dt_bias = torch.full((C,), -3.0, device=device)
+        self._pack(_rand(gen, (R + 2 * N, C), C ** -0.5, dtype, device), _rand(gen, (C, R), R ** -0.5, dtype, device),
+                   torch.log(torch.arange(1, N + 1, device=device, dtype=torch.float32))[None, :].repeat(C, 1))
+        self.w_o = _rand(gen, (W, C), C ** -0.5, dtype, device)
+        return self
+
+    def bind(self, cache, dtype):
+        self.tail = cache.add_state(self.name + ".conv", (self.taps - 1, self.inner)) if self.taps > 1 else None
+        self.state = cache.add_state(self.name + ".ssm", (self.n_state, self.inner))
+
+    def weight_bytes(self):
+        return sum(t.numel() * t.element_size() for t in (self.w_in, self.w_x, self.w_dt, self.w_o))
+
+    def branches(self, h, batch):
+        return [(self.forward(h, batch), None, 1.0)]
+
+    def forward(self, h, batch):
+        C, N, low = self.inner, self.n_state, self.low
+        proj = seqops.gemm_nt(h, self.w_in)                                       # fp32 [x | z]
+        x, xt = seqops.short_conv(proj, 0, self.conv_w, None, self.tail, batch, act=True, bias=self.conv_b, also=h.dtype)
+        small, u = seqops.gemm_nt(xt, self.w_x, lead=low)                         # fp32 [low, padded | B | C]; low once more in the serving format
+        dt = seqops.gemm_nt(u, self.w_dt, bias=self.dt_bias, act="softplus")
+        y = seqops.selective_scan(x, dt, small, low, low + N, proj, C, self.a2, self.d, self.state, batch, h.dtype, seg_len=self.scan_segment)
+        return seqops.gemm_nt(y, self.w_o)
 
 
 class GatedLinearAttention:
@@ -568,6 +754,8 @@ class PlainFF(SideRows):
         return sum(t.numel() * t.element_size() for t in (self.w_up, self.w_down))
 
     def forward(self, h):
+        if self.side_col0 is None:                                                # (the activation in the product's epilogue)
+            return seqops.gemm_nt(seqops.gemm_nt(h, self.w_up, out_dtype=h.dtype, act=self.act), self.w_down)
         z = seqops.gemm_nt(h, self.w_up)                                          # fp32 [up | side rows]
         self.side = (z, self.side_col0)
         return seqops.gemm_nt(seqops.unary_act(z, h.dtype, kind=self.act, cols=self.ff), self.w_down)
@@ -663,15 +851,20 @@ class RoutedExpertsFF(SideRows):
     _side_matrix = "w_router"
 
     def __init__(self, width, ff, experts, top, identity=0, groups=1, keep=1, correction=True, renorm=False, score="softmax", group_top=1,
-                 renorm_eps=0.0, act="silu", act_alpha=1.0, limit=0.0, weight_scale=1.0):
-        """score: "softmax" over all outputs or "sigmoid" of each logit; group_top: a group scores by the sum of its group_top best choice
+                 renorm_eps=0.0, act="silu", act_alpha=1.0, limit=0.0, weight_scale=1.0, router_bias=False, shared_ff=0, shared_gate=False):
+        """score: "softmax" over all outputs, "sigmoid" of each logit, or "chosen" (the largest logits, weighted by a softmax over the chosen
+        ones only); router_bias: tensor router.b (experts + identity) is added to the logits; shared_ff > 0: one more expert `shared` (the
+        same form and activation, its own size) runs for every token and is added, times sigmoid(W_sg h) with shared_gate (tensor shared.sg
+        (1, width)) -- its gate, gate and up rows ride in the router's product; group_top: a group scores by the sum of its group_top best choice
         scores; act: "silu" -- silu(gate) up --, or "swish_clamp" -- g sigmoid(act_alpha g) (u + 1) with g = min(gate, limit),
         u = clamp(up, -limit, limit)"""
-        if score not in ("softmax", "sigmoid") or act not in ("silu", "swish_clamp") or group_top < 1:
+        if score not in seqops.ROUTER_SCORES or act not in ("silu", "swish_clamp") or group_top < 1:
             raise ZLError("experts: unknown score function or activation")
         self.score, self.group_top, self.renorm_eps, self.act, self.act_alpha, self.limit = score, int(group_top), float(renorm_eps), act, \
             float(act_alpha), float(limit)
         self.weight_scale = float(weight_scale)
+        self.has_router_bias, self.shared_ff, self.shared_gate = bool(router_bias), int(shared_ff), bool(shared_gate)
+        self.router_b = self.w_shared_down = None
         total = experts + identity
         if groups < 1 or total % groups or not 1 <= keep <= groups or top > keep * (total // groups):
             raise ZLError("experts: groups must divide the router outputs, and the kept groups must hold `top` outputs")
@@ -688,10 +881,21 @@ class RoutedExpertsFF(SideRows):
         f, w = gate.shape
         return torch.stack([gate.reshape(f // 16, 16, w), up.reshape(f // 16, 16, w)], dim=1).reshape(2 * f, w)
 
+    def _join_shared(self, gate, up, down, sg):
+        """the shared expert's rows join the router's product: [router | shared gates | shared ups | the shared expert's own gate]"""
+        self.shared_col = self.w_router.shape[0]
+        self.w_router = torch.cat([self.w_router, gate, up] + ([sg] if sg is not None else []), dim=0).contiguous()
+        self.w_shared_down = down
+
     def load(self, get, prefix, dtype, device):
         E, f, W = self.experts, self.ff, self.width
         self.w_router = _mat(get, prefix + "router", (E + self.identity, W), dtype, device)
         self.correction = _vec(get, prefix + "correction", E + self.identity, device) if self.has_correction else None
+        self.router_b = _vec(get, prefix + "router.b", E + self.identity, device) if self.has_router_bias else None
+        if self.shared_ff:
+            p, sf = prefix + "shared.", self.shared_ff
+            self._join_shared(_mat(get, p + "gate", (sf, W), dtype, device), _mat(get, p + "up", (sf, W), dtype, device),
+                              _mat(get, p + "down", (W, sf), dtype, device), _mat(get, p + "sg", (1, W), dtype, device) if self.shared_gate else None)
         self.w_gu = torch.empty((E, 2 * f, W), dtype=dtype, device=device)
         self.w_down = torch.empty((E, W, f), dtype=dtype, device=device)
         for e in range(E):
@@ -704,19 +908,24 @@ class RoutedExpertsFF(SideRows):
         E, f, W = self.experts, self.ff, self.width
         self.w_router = _rand(gen, (E + self.identity, W), W ** -0.5, dtype, device)
         self.correction = torch.zeros(E + self.identity, device=device) if self.has_correction else None
+        self.router_b = torch.zeros(E + self.identity, device=device) if self.has_router_bias else None
+        if self.shared_ff:
+            sf = self.shared_ff
+            self._join_shared(_rand(gen, (sf, W), W ** -0.5, dtype, device), _rand(gen, (sf, W), W ** -0.5, dtype, device),
+                              _rand(gen, (W, sf), sf ** -0.5, dtype, device), _rand(gen, (1, W), W ** -0.5, dtype, device) if self.shared_gate else None)
         self.w_gu = _rand(gen, (E, 2 * f, W), W ** -0.5, dtype, device)
         self.w_down = _rand(gen, (E, W, f), f ** -0.5, dtype, device)
         return self
 
     def weight_bytes(self):
-        return sum(t.numel() * t.element_size() for t in (self.w_router, self.w_gu, self.w_down))       # (w_router: with attached side rows)
+        return sum(t.numel() * t.element_size() for t in (self.w_router, self.w_gu, self.w_down, self.w_shared_down) if t is not None)
 
     def forward(self, h):
-        logits = seqops.gemm_nt(h, self.w_router)                                 # fp32 sums of the products [router | side rows]
+        logits = seqops.gemm_nt(h, self.w_router)                                 # fp32 sums of the products [router | shared expert | side rows]
         self.side = (logits, self.side_col0)
         ids, weights = seqops.moe_route(logits, self.correction, self.groups, self.keep, self.top, self.renorm, score=self.score,
                                         group_top=self.group_top, renorm_eps=self.renorm_eps, weight_scale=self.weight_scale,
-                                        n_out=self.experts + self.identity)
+                                        n_out=self.experts + self.identity, logit_bias=self.router_b)
         sorted_tok, slot_pos, tiles, max_tiles, sorted_exp, tm = seqops.moe_align(ids, self.experts, self.tile_m)
         n_slots = ids.numel()
         few = sorted_exp if n_slots <= self.few_rows else None                    # decode steps: weight rows streamed per (row, column)
@@ -727,4 +936,9 @@ class RoutedExpertsFF(SideRows):
             a = seqops.act_mul(seqops.gemm_nt_grouped(h, sorted_tok, self.w_gu, tiles, max_tiles, n_slots, row_expert=few, tile_m=tm), h.dtype,
                                kind=self.act, alpha=self.act_alpha, limit=self.limit, block=16 if self.packed else 0)
         y = seqops.gemm_nt_grouped(a, None, self.w_down, tiles, max_tiles, n_slots, row_expert=few, tile_m=tm)
-        return seqops.moe_combine(y, slot_pos, ids, weights, h, self.experts)
+        if not self.shared_ff:
+            return seqops.moe_combine(y, slot_pos, ids, weights, h, self.experts)
+        s = seqops.gemm_nt(seqops.act_mul(logits, h.dtype, kind=self.act, alpha=self.act_alpha, limit=self.limit, col0=self.shared_col, ff=self.shared_ff),
+                           self.w_shared_down)
+        return seqops.moe_combine(y, slot_pos, ids, weights, h, self.experts, shared=s, gate=logits if self.shared_gate else None,
+                                  g_col=self.shared_col + 2 * self.shared_ff)

@@ -15,13 +15,13 @@ from ._lib import ZLError
 BF16, F32 = 1, 2
 _HERE = os.path.dirname(os.path.abspath(__file__))
 SO_PATH = os.path.join(_HERE, "libzhilight_amd_seq.so")
-SYMBOLS = ["zls_version", "zls_gemm_nt", "zls_embed", "zls_token_shift", "zls_add_scalar_norm", "zls_scalar_norm_rows", "zls_polynorm",
+SYMBOLS = ["zls_version", "zls_gemm_nt", "zls_gemm_nt_act", "zls_embed", "zls_token_shift", "zls_add_scalar_norm", "zls_scalar_norm_rows", "zls_polynorm",
            "zls_latent_store", "zls_latent_attention", "zls_latent_attention_workspace_bytes", "zls_latent_attention_prompt", "zls_gemm_nt_gather",
-           "zls_conv_silu", "zls_conv_tail_update", "zls_ssm_scan", "zls_ssm_scan_workspace_bytes", "zls_gated_group_norm", "zls_layer_norm",
+           "zls_conv_silu", "zls_ssm_scan", "zls_ssm_scan_workspace_bytes", "zls_selective_scan", "zls_selective_scan_workspace_bytes", "zls_gated_group_norm", "zls_layer_norm",
            "zls_add_layer_norm", "zls_rope_norm_store", "zls_window_attention", "zls_window_attention_prompt", "zls_head_mix_gate", "zls_decay_scan", "zls_exp_gates",
            "zls_linear_attn_finish", "zls_moe_route", "zls_moe_align", "zls_gemm_nt_grouped", "zls_silu_mul", "zls_moe_combine", "zls_rms_norm",
-           "zls_add_rms_norm", "zls_scale_softcap", "zls_act_mul", "zls_short_conv", "zls_short_conv_tail", "zls_lowrank_decay", "zls_latent_rope_store",
-           "zls_streams_norm", "zls_streams_update", "zls_unary_act"]
+           "zls_add_rms_norm", "zls_scale_softcap", "zls_act_mul", "zls_short_conv", "zls_lowrank_decay", "zls_latent_rope_store",
+           "zls_streams_norm", "zls_streams_update", "zls_unary_act", "zls_add_branches"]
 _STATUS = {-1: "invalid argument (null pointer / non-positive size)", -2: "shape not supported", -3: "dtype not supported",
            -4: "exceeds a hardware limit"}
 
@@ -36,7 +36,13 @@ class Batch(C.Structure):
 class ScoreForm(C.Structure):
     """zls_score_form_t"""
     _fields_ = [("head_scale", C.c_void_p), ("softcap", C.c_float), ("bias", C.c_void_p), ("bias_rows", C.c_int32), ("offset", C.c_void_p),
-                ("chunk", C.c_int32), ("sigmoid", C.c_int32)]
+                ("chunk", C.c_int32), ("sigmoid", C.c_int32), ("slope", C.c_void_p)]
+
+
+class HeadPrep(C.Structure):
+    """zls_head_prep_t"""
+    _fields_ = [("whole_norm", C.c_int32), ("q_w", C.c_void_p), ("k_w", C.c_void_p), ("temp_coef", C.c_float), ("temp_every", C.c_int32),
+                ("x_col0", C.c_int32), ("x_heads", C.c_int32), ("x_dim", C.c_int32), ("x_rot", C.c_int32), ("x_freq", C.c_void_p)]
 
 
 _lib = None
@@ -53,6 +59,7 @@ def lib():
             getattr(l, name)
         l.zls_latent_attention_workspace_bytes.restype = C.c_int64
         l.zls_ssm_scan_workspace_bytes.restype = C.c_int64
+        l.zls_selective_scan_workspace_bytes.restype = C.c_int64
         _lib = l
     return _lib
 
@@ -178,22 +185,27 @@ class RaggedBatch:
         return self._windowed[window]
 
 
-def gemm_nt(x, w, out=None, out_dtype=torch.float32):
-    """x (m, k) . w (n, k)^T -> (m, n); x and w in the serving format, the result fp32 (or that format)."""
-    _cuda(w)
+def gemm_nt(x, w, out=None, out_dtype=torch.float32, bias=None, act=None, lead=0):
+    """act(x (m, k) . w (n, k)^T + bias) -> (m, n); x and w in the serving format, the result fp32 (or that format); bias fp32 (n) or None,
+    act one of UNARY_ACTS or None.  lead > 0: returns (result, its leading `lead` columns once more in the serving format)"""
+    _cuda(w, bias)
+    _f32(bias)
     if x.dim() != 2 or x.stride(1) != 1 or not x.is_cuda:
         raise ZLError("gemm_nt: x must be a device matrix with unit column stride")
     m, k = x.shape
     n = w.shape[0]
     if w.shape[1] != k or w.dtype != x.dtype:
         raise ZLError("gemm_nt: size K / dtype mismatch")
+    if bias is not None and bias.numel() != n:
+        raise ZLError("gemm_nt: one bias per output column")
     if out is None:
         out = torch.empty((m, n), dtype=out_dtype, device=x.device)
     elif out.shape != (m, n) or not out.is_contiguous():
         raise ZLError("gemm_nt: wrong output")
-    check(lib().zls_gemm_nt(_p(x), _i(x.stride(0)), _p(w), _p(out), _i(n), _i(m), _i(n), _i(k), C.c_int(dt_code(x.dtype)),
-                            C.c_int(dt_code(out.dtype)), _stream()), "gemm_nt")
-    return out
+    y2 = torch.empty((m, lead), dtype=x.dtype, device=x.device) if lead > 0 else None
+    check(lib().zls_gemm_nt_act(_p(x), _i(x.stride(0)), _p(w), _p(bias), C.c_int(-1 if act is None else UNARY_ACTS[act]), _p(out), _i(n), _p(y2),
+                                _i(lead), _i(lead), _i(m), _i(n), _i(k), C.c_int(dt_code(x.dtype)), C.c_int(dt_code(out.dtype)), _stream()), "gemm_nt")
+    return (out, y2) if lead > 0 else out
 
 
 def embed(tokens, table, pos_table, scale, batch, out=None):
@@ -320,23 +332,13 @@ def latent_attention(q, q_col0, gate, g_col0, w_uk, w_uv, sink, cache, batch, sc
 
 
 def conv_silu(proj, col0, w, bias, tail, batch):
-    """causal convolution + SiLU over `channels` columns of proj from col0, then the carried tail moves on (two launches)"""
-    _cuda(proj, w, bias, tail)
-    _f32(proj, w, bias, tail)
-    channels, taps = w.shape
-    if tail is not None and tuple(tail.shape[1:]) != (taps - 1, channels):
-        raise ZLError("conv_silu: tail must be (slots, taps - 1, channels)")
-    out = torch.empty((batch.n_tok, channels), dtype=torch.float32, device=proj.device)
-    check(lib().zls_conv_silu(_p(proj), _i(proj.shape[1]), _i(col0), _p(w), _p(bias), _p(tail), _i(channels), _i(taps), batch.ref, _p(out),
-                              _stream()), "conv_silu")
-    check(lib().zls_conv_tail_update(_p(proj), _i(proj.shape[1]), _i(col0), _p(tail), _i(channels), _i(taps), batch.ref, _stream()),
-          "conv_tail_update")
-    return out
+    """causal convolution + SiLU over `channels` columns of proj from col0; the carried tail moves on"""
+    return short_conv(proj, col0, w, None, tail, batch, act=True, bias=bias)
 
 
-def short_conv(proj, col0, w, in_bias, tail, batch, act=False, bias=None):
+def short_conv(proj, col0, w, in_bias, tail, batch, act=False, bias=None, also=None):
     """causal convolution over `channels` columns of proj from col0: in_bias joins every input, `bias` the result, act: SiLU; the carried
-    tail moves on (two launches)"""
+    tail moves on.  also (a dtype): returns (fp32 result, the result in that format)"""
     _cuda(proj, w, bias, in_bias, tail)
     _f32(proj, w, bias, in_bias, tail)
     channels, taps = w.shape
@@ -346,11 +348,10 @@ def short_conv(proj, col0, w, in_bias, tail, batch, act=False, bias=None):
         if t is not None and t.numel() != channels:
             raise ZLError("short_conv: one bias per channel")
     out = torch.empty((batch.n_tok, channels), dtype=torch.float32, device=proj.device)
+    out_t = torch.empty_like(out, dtype=also) if also not in (None, torch.float32) else None
     check(lib().zls_short_conv(_p(proj), _i(proj.shape[1]), _i(col0), _p(w), _p(bias), _p(in_bias), C.c_int(int(act)), _p(tail), _i(channels),
-                               _i(taps), batch.ref, _p(out), _stream()), "short_conv")
-    check(lib().zls_short_conv_tail(_p(proj), _i(proj.shape[1]), _i(col0), _p(in_bias), _p(tail), _i(channels), _i(taps), batch.ref, _stream()),
-          "short_conv_tail")
-    return out
+                               _i(taps), batch.ref, _p(out), _p(out_t), C.c_int(F32 if out_t is None else dt_code(also)), _stream()), "short_conv")
+    return out if also is None else (out, out if out_t is None else out_t)
 
 
 SCAN_SEGMENT = 256      # tokens per segment of a long portion (ssm_scan)
@@ -369,6 +370,30 @@ def ssm_scan(xbc, proj, dt_col0, dt_bias, a_log, d, state, heads, vdim, n_state,
                                                                 _i(n_state))) // 4, dtype=torch.float32, device=xbc.device)
     check(lib().zls_ssm_scan(_p(xbc), _p(proj), _i(proj.shape[1]), _i(dt_col0), _p(dt_bias), _p(a_log), _p(d), _p(state), _i(heads), _i(vdim),
                              _i(n_state), _i(groups), batch.ref, _p(y), _p(ws), _i(seg_len), _stream()), "ssm_scan")
+    return y
+
+
+SELECTIVE_SEGMENT = 128     # tokens per segment of a long portion (selective_scan)
+
+
+def selective_scan(x, dt, bc, b_col0, c_col0, zrow, z_col0, a2, d, state, batch, dtype, seg_len=None):
+    """S[n][c] <- 2^(dt_c a2[n][c]) S[n][c] + dt_c x_c B_n; (sum_n S[n][c] C_n + d_c x_c) * silu(z_c) in `dtype` (n_tok, inner)"""
+    _cuda(x, dt, bc, zrow, a2, d, state)
+    _f32(x, dt, bc, zrow, a2, d, state)
+    n_tok, inner = x.shape
+    n_state = a2.shape[0]
+    if dt.shape != x.shape or tuple(a2.shape) != (n_state, inner) or d.numel() != inner or tuple(state.shape[1:]) != (n_state, inner) or \
+            n_tok != batch.n_tok or bc.shape[0] != n_tok or zrow.shape[0] != n_tok:
+        raise ZLError("selective_scan: shapes")
+    y = torch.empty((n_tok, inner), dtype=dtype, device=x.device)
+    seg_len = SELECTIVE_SEGMENT if seg_len is None else seg_len
+    ws = None
+    if seg_len > 0 and batch.c.max_count > seg_len:
+        ws = torch.empty(int(lib().zls_selective_scan_workspace_bytes(_i(batch.n_seq), _i(batch.c.max_count), _i(seg_len), _i(inner), _i(n_state))) // 4,
+                         dtype=torch.float32, device=x.device)
+    check(lib().zls_selective_scan(_p(x), _p(dt), _p(bc), _i(bc.shape[1]), _i(b_col0), _i(c_col0), _p(zrow), _i(zrow.shape[1]), _i(z_col0), _p(a2),
+                                   _p(d), _p(state), _i(inner), _i(n_state), batch.ref, _p(y), _p(ws), _i(seg_len), C.c_int(dt_code(dtype)),
+                                   _stream()), "selective_scan")
     return y
 
 
@@ -435,6 +460,31 @@ def add_rms_norm(x, y, eps, next_weight=None, dtype=None, around_zero=False):
     return h2
 
 
+# ---- sub-layers that run side by side ----------------------------------------------------------------------------------------------------
+class Branch(C.Structure):
+    """zls_branch_t"""
+    _fields_ = [("y", C.c_void_p), ("w", C.c_void_p), ("coef", C.c_float)]
+
+
+def add_branches(x, branches, eps, dtype, weight1=None, weight2=None, xt=None):
+    """x += sum of coef * N(y) over branches = [(y, w or None, coef)] in place (w None: y as it is; no branches: x stays); returns (h1, h2) =
+    the RMS norms of the new x with weight1 / weight2 in `dtype` (None without the weight); xt: a (rows, width) view of unit column stride
+    that receives the new x in its own format"""
+    _cuda(x, weight1, weight2, *[t for b in branches for t in b[:2]])
+    _f32(x, weight1, weight2, *[t for b in branches for t in b[:2]])
+    rows, width = x.shape
+    for y, w, _ in branches:
+        if y.shape != x.shape or (w is not None and w.numel() != width):
+            raise ZLError("add_branches: shape mismatch")
+    if xt is not None and (xt.shape != x.shape or xt.stride(1) != 1 or xt.dtype != dtype or not xt.is_cuda):
+        raise ZLError("add_branches: xt must be rows of x's shape in the serving format")
+    h1, h2 = (torch.empty((rows, width), dtype=dtype, device=x.device) if w is not None else None for w in (weight1, weight2))
+    arr = (Branch * max(1, len(branches)))(*[Branch(y.data_ptr(), 0 if w is None else w.data_ptr(), float(c)) for y, w, c in branches])
+    check(lib().zls_add_branches(_p(x), arr, _i(len(branches)), _f(eps), _i(rows), _i(width), _p(weight1), _p(h1), _p(weight2), _p(h2), _p(xt),
+                                 _i(0 if xt is None else xt.stride(0)), C.c_int(dt_code(dtype)), _stream()), "add_branches")
+    return h1, h2
+
+
 # ---- a residual kept as several streams ------------------------------------------------------------------------------------------------
 def streams_norm(xs, n, read_coef, weight, eps, dtype, rows=None, around_zero=False):
     """N(sum_s read_coef[s] x_s) of the rows `rows` (None: all) in `dtype`.  xs fp32: (n_tok, n, width), or (n_tok, width) read as n equal
@@ -473,7 +523,7 @@ def streams_update(src, dst, n, y, mix, out_coef, gate=None, g_col0=0, gate_bias
     return h
 
 
-UNARY_ACTS = {"relu2": 0, "gelu_tanh": 1, "silu": 2}
+UNARY_ACTS = {"relu2": 0, "gelu_tanh": 1, "silu": 2, "softplus": 3}
 
 
 def unary_act(z, dtype, kind="relu2", cols=None):
@@ -497,16 +547,36 @@ def scale_softcap(z, scale, cap):
 
 
 # ---- softmax attention over paged keys and values -------------------------------------------------------------------------------------------
+def head_prep(whole_norm=False, q_w=None, k_w=None, temp=None, extra=None):
+    """The optional parts of rope_norm_store: one norm over all query (key) heads of a token with a weight per number (q_w, k_w fp32), before
+    the rotation; temp = (coef, every): queries times 1 + coef ln(floor((p + 1) / every) + 1); extra = (column, heads, dim, rotated
+    coordinates, frequencies): further heads of the same rows that are rotated in place.  Keeps the tensors alive."""
+    _cuda(q_w, k_w)
+    _f32(q_w, k_w)
+    coef, every = temp if temp else (0.0, 0)
+    col, heads, dim, rot, freq = extra if extra else (0, 0, 0, 0, None)
+    _cuda(freq)
+    _f32(freq)
+    if freq is not None and freq.numel() != rot // 2 or (rot and freq is None):
+        raise ZLError("head_prep: one frequency per rotated pair")
+    h = HeadPrep(int(bool(whole_norm)), 0 if q_w is None else q_w.data_ptr(), 0 if k_w is None else k_w.data_ptr(), float(coef), int(every),
+                 int(col), int(heads), int(dim), int(rot), 0 if freq is None else freq.data_ptr())
+    h.keep, h.sizes = (q_w, k_w, freq), (0 if q_w is None else q_w.numel(), 0 if k_w is None else k_w.numel())
+    return h
+
+
 def rope_norm_store(proj, q_col0, k_col0, v_col0, heads, kv_heads, dim, vdim, qk_freq, rot_dims, v_freq, eps, qk_norm, batch, k_cache, v_cache,
-                    interleaved=False, vmix=None, q_norm_w=None, k_norm_w=None):
+                    interleaved=False, vmix=None, q_norm_w=None, k_norm_w=None, prep=None):
     """rotate / norm the queries in place in proj; rotate / norm the keys and turn the values into the paged planes (None: queries only).
     interleaved: rotated pairs are neighbours (2i, 2i + 1).  vmix = (src, col0, lam): values <- (1 - lam) values + lam src[t][col0 ..].
-    q_norm_w / k_norm_w: fp32 (dim) weights of the norm, shared by the heads"""
+    q_norm_w / k_norm_w: fp32 (dim) weights of the norm, shared by the heads; prep: head_prep()"""
     _cuda(proj, qk_freq, v_freq, k_cache, v_cache, q_norm_w, k_norm_w)
     _f32(proj, qk_freq, v_freq, q_norm_w, k_norm_w)
     for t in (q_norm_w, k_norm_w):
         if t is not None and (t.numel() != dim or not qk_norm):
             raise ZLError("rope_norm_store: a norm weight has one number per coordinate of a head")
+    if prep is not None and (prep.sizes[0] not in (0, heads * dim) or prep.sizes[1] not in (0, kv_heads * dim)):
+        raise ZLError("rope_norm_store: the weights of a whole-row norm have one number per coordinate of all heads")
     vsrc, vcol, vlam = vmix if vmix is not None else (None, 0, 0.0)
     if vsrc is not None and (vsrc.dtype != torch.float32 or vsrc.dim() != 2 or vsrc.stride(1) != 1 or vsrc.shape[0] != batch.n_tok):
         raise ZLError("rope_norm_store: the blended values are fp32 rows, one per token")
@@ -520,23 +590,25 @@ def rope_norm_store(proj, q_col0, k_col0, v_col0, heads, kv_heads, dim, vdim, qk
     code = dt_code(k_cache.dtype) if k_cache is not None else F32
     check(lib().zls_rope_norm_store(_p(proj), _i(proj.shape[1]), _i(q_col0), _i(k_col0), _i(v_col0), _i(heads), _i(kv_heads), _i(dim), _i(vdim),
                                     _p(qk_freq), _i(rot_dims), _p(v_freq), _f(eps), C.c_int(int(qk_norm)), C.c_int(int(interleaved)), _p(vsrc),
-                                    _i(0 if vsrc is None else vsrc.stride(0)), _i(vcol), _f(vlam), _p(q_norm_w), _p(k_norm_w), batch.ref, _p(k_cache), _p(v_cache),
+                                    _i(0 if vsrc is None else vsrc.stride(0)), _i(vcol), _f(vlam), _p(q_norm_w), _p(k_norm_w),
+                                    C.byref(prep) if prep is not None else None, batch.ref, _p(k_cache), _p(v_cache),
                                     C.c_int(code), _stream()), "rope_norm_store")
 
 
-def score_form(heads, head_scale=None, softcap=0.0, bias=None, offset=None, chunk=0, sigmoid=False):
+def score_form(heads, head_scale=None, softcap=0.0, bias=None, offset=None, chunk=0, sigmoid=False, slope=None):
     """The optional score form of window_attention: per-head factor (heads), tanh cap, distance bias fp32 (heads, rows) -- row min(p - j,
-    rows - 1) --, chunked visibility, sigmoid weights with a per-head offset.  Returns an object that keeps the tensors alive."""
-    _cuda(head_scale, bias, offset)
-    _f32(head_scale, bias, offset)
-    for t in (head_scale, offset):
+    rows - 1) --, linear distance bias -slope[head] (p - j), chunked visibility, sigmoid weights with a per-head offset.  Returns an object that keeps the tensors alive."""
+    _cuda(head_scale, bias, offset, slope)
+    _f32(head_scale, bias, offset, slope)
+    for t in (head_scale, offset, slope):
         if t is not None and t.numel() != heads:
             raise ZLError("score_form: one number per head")
     if bias is not None and (bias.dim() != 2 or bias.shape[0] != heads):
         raise ZLError("score_form: the distance bias is (heads, rows)")
     f = ScoreForm(0 if head_scale is None else head_scale.data_ptr(), float(softcap or 0.0), 0 if bias is None else bias.data_ptr(),
-                  0 if bias is None else bias.shape[1], 0 if offset is None else offset.data_ptr(), int(chunk), int(bool(sigmoid)))
-    f.keep = (head_scale, bias, offset)
+                  0 if bias is None else bias.shape[1], 0 if offset is None else offset.data_ptr(), int(chunk), int(bool(sigmoid)),
+                  0 if slope is None else slope.data_ptr())
+    f.keep = (head_scale, bias, offset, slope)
     return f
 
 
@@ -658,24 +730,27 @@ def linear_attn_finish(y, norm_col, q_scale, m_vals, den_eps, heads, vdim, norm_
 # ---- mixture of experts ------------------------------------------------------------------------------------------------------------------
 MOE_TILE = 64           # rows of an expert's tile in the grouped products; 128 when the average expert gets at least MOE_BIG_SHARE rows
 MOE_BIG_SHARE = 256
+ROUTER_SCORES = {"softmax": 0, "sigmoid": 1, "chosen": 2}
 
 
-def moe_route(logits, correction, groups, keep, top, renorm=False, score="softmax", group_top=1, renorm_eps=0.0, weight_scale=1.0, n_out=None):
-    """n_out: the router's outputs are the leading n_out columns of wider rows (None: all columns)"""
-    _cuda(logits, correction)
-    _f32(logits, correction)
+def moe_route(logits, correction, groups, keep, top, renorm=False, score="softmax", group_top=1, renorm_eps=0.0, weight_scale=1.0, n_out=None,
+              logit_bias=None):
+    """score: softmax over all outputs, sigmoid of each, or "chosen" -- the choice is among the logits, the weights are a softmax over the
+    chosen ones; logit_bias fp32 (n_out) is added to the logits first.  n_out: the router's outputs are the leading n_out columns of wider rows (None: all columns)"""
+    _cuda(logits, correction, logit_bias)
+    _f32(logits, correction, logit_bias)
     n_tok = logits.shape[0]
     n_out = logits.shape[1] if n_out is None else int(n_out)
     if n_out > logits.shape[1]:
         raise ZLError("moe_route: more router outputs than columns")
-    if correction is not None and correction.numel() != n_out:
-        raise ZLError("moe_route: one correction per router output")
+    if any(t is not None and t.numel() != n_out for t in (correction, logit_bias)):
+        raise ZLError("moe_route: one correction / bias per router output")
     ids = torch.empty((n_tok, top), dtype=torch.int32, device=logits.device)
     weights = torch.empty((n_tok, top), dtype=torch.float32, device=logits.device)
-    if score not in ("softmax", "sigmoid"):
-        raise ZLError("moe_route: scores are softmax or sigmoid")
-    check(lib().zls_moe_route(_p(logits), _i(logits.stride(0)), _i(n_tok), _i(n_out), _p(correction), _i(groups), _i(keep), _i(top), C.c_int(int(renorm)),
-                              C.c_int(1 if score == "sigmoid" else 0), _i(group_top), _f(renorm_eps), _f(weight_scale), _p(ids), _p(weights), _stream()),
+    if score not in ROUTER_SCORES:
+        raise ZLError("moe_route: scores are softmax, sigmoid or chosen")
+    check(lib().zls_moe_route(_p(logits), _i(logits.stride(0)), _i(n_tok), _i(n_out), _p(logit_bias), _p(correction), _i(groups), _i(keep), _i(top), C.c_int(int(renorm)),
+                              C.c_int(ROUTER_SCORES[score]), _i(group_top), _f(renorm_eps), _f(weight_scale), _p(ids), _p(weights), _stream()),
           "moe_route")
     return ids, weights
 
@@ -725,22 +800,30 @@ def silu_mul(gu, dtype):
     return out
 
 
-def act_mul(gu, dtype, kind="silu", alpha=1.0, limit=0.0, block=0):
-    """act(gate, up) of fp32 rows [gates | ups] (block 0) or blocks of `block` gates followed by their ups; see ACT_KINDS"""
+def act_mul(gu, dtype, kind="silu", alpha=1.0, limit=0.0, block=0, col0=0, ff=None):
+    """act(gate, up) of fp32 rows [gates | ups] (block 0) or blocks of `block` gates followed by their ups; see ACT_KINDS.  ff: the 2 ff
+    columns from col0 of wider rows (None: all columns)"""
     _cuda(gu)
     _f32(gu)
-    rows, two_ff = gu.shape
-    out = torch.empty((rows, two_ff // 2), dtype=dtype, device=gu.device)
-    check(lib().zls_act_mul(_p(gu), _i(rows), _i(two_ff // 2), C.c_int(ACT_KINDS[kind]), _f(alpha), _f(limit), _i(block), _p(out),
-                            C.c_int(dt_code(dtype)), _stream()), "act_mul")
+    rows, ld = gu.shape
+    ff = ld // 2 if ff is None else ff
+    if col0 < 0 or col0 + 2 * ff > ld:
+        raise ZLError("act_mul: columns")
+    out = torch.empty((rows, ff), dtype=dtype, device=gu.device)
+    check(lib().zls_act_mul(C.c_void_p(gu.data_ptr() + 4 * col0), _i(ld), _i(rows), _i(ff), C.c_int(ACT_KINDS[kind]), _f(alpha), _f(limit), _i(block),
+                            _p(out), C.c_int(dt_code(dtype)), _stream()), "act_mul")
     return out
 
 
-def moe_combine(y, slot_pos, ids, weights, h, n_experts):
-    _cuda(y, slot_pos, ids, weights, h)
-    _f32(y, weights)
+def moe_combine(y, slot_pos, ids, weights, h, n_experts, shared=None, gate=None, g_col=0):
+    """the weighted sum of every token's picks; shared fp32 (n_tok, width): a shared expert's rows, added times sigmoid(gate[:, g_col])"""
+    _cuda(y, slot_pos, ids, weights, h, shared, gate)
+    _f32(y, weights, shared, gate)
     n_tok, top = ids.shape
+    if shared is not None and tuple(shared.shape) != (n_tok, h.shape[1]):
+        raise ZLError("moe_combine: the shared expert's rows do not fit")
     out = torch.empty((n_tok, h.shape[1]), dtype=torch.float32, device=h.device)
-    check(lib().zls_moe_combine(_p(y), _p(slot_pos), _p(ids), _p(weights), _p(h), _i(n_tok), _i(top), _i(n_experts), _i(h.shape[1]), _p(out),
-                                C.c_int(dt_code(h.dtype)), _stream()), "moe_combine")
+    check(lib().zls_moe_combine(_p(y), _p(slot_pos), _p(ids), _p(weights), _p(h), _i(n_tok), _i(top), _i(n_experts), _i(h.shape[1]), _p(shared),
+                                _p(gate), _i(0 if gate is None else gate.shape[1]), _i(g_col), _p(out), C.c_int(dt_code(h.dtype)), _stream()),
+          "moe_combine")
     return out
