@@ -223,7 +223,9 @@ def random_weights(cfg, seed=0, fixed_choice=False):
     """every tensor the configuration asks for, bf16-representable values (both serving formats start from the same numbers).
     fixed_choice: the routers read ONE reserved coordinate of the residual only -- coordinate 0 of the embedding holds a number whose sign
     and size the token decides, no sub-layer writes to it and the loop's entry copies it -- with evenly spaced multiples per expert, so
-    that the order of the logits is one fixed order or its reverse, with wide gaps: no choice is a close call under a rounded router input."""
+    that the order of the logits is one fixed order or its reverse, with wide gaps: no choice is a close call under a rounded router input.
+    The retention's key matrices then also lean towards its query matrices: a sequence's first output is (q . k) v / rms, whose SIGN hangs on
+    a product that random matrices let come close to zero."""
     g = torch.Generator().manual_seed(seed)
     W, scale = cfg["width"], float(cfg["embedding"]["scale"])
     sd = {}
@@ -236,7 +238,7 @@ def random_weights(cfg, seed=0, fixed_choice=False):
 
     mat("embed", cfg["vocab"], W, 1.5 / scale)
     if fixed_choice:
-        size = (2.0 + 2.0 * torch.rand(cfg["vocab"], generator=g)) / scale
+        size = (4.0 + 4.0 * torch.rand(cfg["vocab"], generator=g)) / scale
         sd["embed"][:, 0] = torch.where(torch.arange(cfg["vocab"]) % 3 == 0, -size, size).to(torch.bfloat16)
     mat("head", cfg["vocab"], W)
     vec("final.norm", W, 0.2, 1.0)
@@ -269,6 +271,8 @@ def random_weights(cfg, seed=0, fixed_choice=False):
             H, d, e = r["heads"], r["dim"], r["vdim"]
             for n, rows in (("q", H * d), ("k", H * d), ("v", H * e), ("g", H * e)):
                 mat(p + "mix.right." + n, rows, W)
+            if fixed_choice:
+                sd[p + "mix.right.k"] = (0.8 * sd[p + "mix.right.q"].float() + 0.5 * sd[p + "mix.right.k"].float()).to(torch.bfloat16)
             mat(p + "mix.right.o", W, H * e)
             vec(p + "mix.left.out", W, 0.2, 1.0)
             vec(p + "mix.right.out", W, 0.2, 0.8)
@@ -285,7 +289,7 @@ def random_weights(cfg, seed=0, fixed_choice=False):
         vec(p + "mlp.router.b", E, 0.5)
         if fixed_choice:
             q = torch.zeros(E, W)
-            q[:, 0] = 0.8 * torch.randperm(E, generator=g).double() - 0.4 * E
+            q[:, 0] = 1.6 * torch.randperm(E, generator=g).double() - 0.8 * E
             sd[p + "mlp.router"] = q.to(torch.bfloat16)
             sd[p + "mlp.router.b"] = (0.1 * sd[p + "mlp.router.b"].float()).to(torch.bfloat16)
         names = [(f"e{j}.", f["expert"]["ff"]) for j in range(E)] + ([("shared.", f["shared"]["ff"])] if f.get("shared") else [])
