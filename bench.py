@@ -20,12 +20,14 @@ fields, `roofline` (the W4A16 GEMV kernel: algorithmic bytes / HIP-event time, v
     python bench.py --retotar 1b,8b [--seq 2048]
     python bench.py --gutivik 1b,8b [--seq 2048]
     python bench.py --gaparax 1b,8b [--seq 2048] [--only TEXT]
+    python bench.py --zasazen 1b,8b [--seq 2048] [--only TEXT]
 
 is a different measurement with its own JSON line: prefill / decode throughput of the ragged-step engine's latent-attention, state-space
 and hybrid stacks (zhilight_amd/tupitar.py) beside the dense bf16 Llama-shaped stack of equal width, 4 layers each, random weights;
 --retotar the same for the Retotar stacks (zhilight_amd/retotar.py) beside the Tupitar hybrid of equal width.
 --gutivik the same for the Gutivik stacks (zhilight_amd/gutivik.py) beside Retotar stacks of equal width.
 --gaparax the same for the Gaparax stacks (zhilight_amd/gaparax.py) beside Gutivik stacks of equal width.
+--zasazen the same for the Zasazen stacks (zhilight_amd/zasazen.py) beside Gutivik, Retotar and Tupitar stacks of equal width.
 """
 import argparse
 import json
@@ -785,8 +787,70 @@ def bench_gaparax(args, dev):
     print(json.dumps({"metric": "gaparax_throughput", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "layers": 4, "results": results}))
 
 
+ZASAZEN_BENCH_SIZES = {
+    # name: width; attention heads / key-value heads x head size; retention heads x key size x value size; state-space channels, states, rank of
+    #       the step-size projection, taps; experts x their ff, picks, the shared expert's ff; the dense feed-forward's ff (two matrices that
+    #       hold what the picked experts' three hold).  Head counts, sizes and experts are those of the sizes of the same name above.
+    "1b": dict(width=2048, heads=16, kv_heads=4, dim=128, r_heads=16, r_dim=128, r_vdim=128, inner=4096, state=16, dt_rank=128, taps=4,
+               experts=16, ff=1360, top=4, shared_ff=1360, dense_ff=8160),
+    "8b": dict(width=4096, heads=32, kv_heads=8, dim=128, r_heads=32, r_dim=128, r_vdim=128, inner=8192, state=16, dt_rank=256, taps=4,
+               experts=32, ff=2384, top=4, shared_ff=2384, dense_ff=14304),
+}
+
+
+def bench_zasazen(args, dev):
+    """--zasazen: prefill and decode throughput of Zasazen stacks (zhilight_amd/zasazen.py: mixer and feed-forward side by side; attention with
+    a linear distance bias beside a retention layer; a selective state space with a decay per channel and state; experts with a gated shared
+    expert; looped layers) beside the closest existing models of equal width -- Gutivik's attention stack, Retotar's decayed linear attention
+    stack, Tupitar's Mamba-2 stack --, 4 layer runs each, random weights, bf16, eager launches.  One JSON line."""
+    from zhilight_amd.gutivik import GutivikConfig, GutivikLayerConfig, GutivikModel
+    from zhilight_amd.retotar import RetotarConfig, RetotarLayerConfig, RetotarModel
+    from zhilight_amd.tupitar import TupitarConfig, TupitarLayerConfig, TupitarModel
+    from zhilight_amd.zasazen import ZasazenConfig, ZasazenLayerConfig, ZasazenModel
+    seq, vocab, results = args.seq, 32000, []
+
+    def measure(label, name, build):
+        if args.only and args.only not in label:
+            return
+        model = build().init_random(1)
+        _measure_ragged(results, label, name, model, seq, vocab)
+
+    for name in args.zasazen.split(","):
+        z = ZASAZEN_BENCH_SIZES[name]
+        mlp = dict(kind="moe", expert=dict(ff=z["ff"]), router=dict(experts=z["experts"], top=z["top"]), shared=dict(ff=z["shared_ff"]))
+        dense = dict(kind="dense", ff=z["dense_ff"])
+        par = dict(left=dict(heads=z["heads"], kv_heads=z["kv_heads"], dim=z["dim"], vdim=z["dim"], scale=z["dim"] ** -0.5, q_temp=dict(coef=0.1, every=512)),
+                   right=dict(heads=z["r_heads"], dim=z["r_dim"], vdim=z["r_vdim"], decay=[1.0 - 2.0 ** -(3 + 5 * h / z["r_heads"]) for h in range(z["r_heads"])],
+                              rot=dict(dims=z["r_dim"], base=1e4)))
+        ssm = dict(inner=z["inner"], state=z["state"], dt_rank=z["dt_rank"], conv=z["taps"])
+        P, Pd = ZasazenLayerConfig("parallel", par, mlp), ZasazenLayerConfig("parallel", par, dense)
+        M, Md = ZasazenLayerConfig("mamba1", ssm, mlp), ZasazenLayerConfig("mamba1", ssm, dense)
+        for label, layers, loop in (("parallel x4", [P] * 4, None), ("mamba1 x4, dense", [Md] * 4, None), ("hybrid (m, p, p, m), dense / experts", [Md, P, Pd, M], None),
+                                    ("hybrid (m, p) run twice, dense / experts", [Md, P], (0, 2, 2))):
+            measure("zasazen " + label, name, lambda: ZasazenModel(ZasazenConfig(vocab, z["width"], 1.0, 1e-6, loop, 1 << 24, layers), "bfloat16", dev))
+        g = GUTIVIK_BENCH_SIZES[name]
+        gmlp = dict(kind="moe", expert=dict(ff=g["ff"], limit=7.0), router=dict(experts=g["experts"], top=g["top"],
+                                                                                groups=dict(count=g["groups"], keep=g["keep_groups"])))
+        gatt = dict(heads=g["heads"], kv_heads=g["kv_heads"], dim=g["dim"], vdim=g["dim"], scale=g["dim"] ** -0.5, rot=dict(dims=g["rot"], base=1e6))
+        measure("gutivik attention x4, no window", name, lambda: GutivikModel(
+            GutivikConfig(vocab, z["width"], 1e-6, 1.0, 0.0, 1 << 24, [GutivikLayerConfig("attention", gatt, gmlp)] * 4), "bfloat16", dev))
+        r = RETOTAR_BENCH_SIZES[name]
+        rmlp = dict(kind="moe", expert=dict(ff=r["ff"]), router=dict(experts=r["experts"], identity=0, top=r["top"]))
+        rlin = dict(heads=r["l_heads"], dim=r["l_dim"], vdim=r["l_vdim"], decay=par["right"]["decay"])
+        measure("retotar lightning x4", name, lambda: RetotarModel(
+            RetotarConfig(vocab, z["width"], 1.0, 1e-6, 1 << 24, [RetotarLayerConfig("lightning", rlin, rmlp)] * 4), "bfloat16", dev))
+        t = SEQ_BENCH_SIZES[name]
+        tssm = dict(heads=t["m_heads"], vdim=t["m_vdim"], state=t["state"], groups=t["groups"], conv=4, norm_groups=t["groups"])
+        measure("tupitar mamba2 x4, dense", name, lambda: TupitarModel(
+            TupitarConfig(vocab, z["width"], seq + 64, 1.0, 1e-6, [TupitarLayerConfig("mamba2", tssm, dict(ff=t["ff"], kind="dense"))] * 4), "bfloat16", dev))
+    print(json.dumps({"metric": "zasazen_throughput", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "layers": 4, "results": results}))
+
+
 def main():
     ap = argparse.ArgumentParser()
+    ap.add_argument("--zasazen", default="", metavar="SIZES",
+                    help="instead of the default workload: prefill / decode throughput of Zasazen stacks beside Gutivik, Retotar and Tupitar "
+                         "stacks of equal width; comma-separated sizes of " + ", ".join(ZASAZEN_BENCH_SIZES))
     ap.add_argument("--gaparax", default="", metavar="SIZES",
                     help="instead of the default workload: prefill / decode throughput of Gaparax stacks beside Gutivik stacks of equal "
                          "width; comma-separated sizes of " + ", ".join(GAPARAX_BENCH_SIZES))
@@ -796,7 +860,7 @@ def main():
     ap.add_argument("--gutivik", default="", metavar="SIZES",
                     help="instead of the default workload: prefill / decode throughput of Gutivik stacks beside Retotar stacks of equal "
                          "width; comma-separated sizes of " + ", ".join(GUTIVIK_BENCH_SIZES))
-    ap.add_argument("--only", default="", metavar="TEXT", help="with --gutivik / --gaparax: only the stacks whose label contains TEXT (e.g. for a kernel trace of one model)")
+    ap.add_argument("--only", default="", metavar="TEXT", help="with --gutivik / --gaparax / --zasazen: only the stacks whose label contains TEXT (e.g. for a kernel trace of one model)")
     ap.add_argument("--mixers", default="", metavar="SIZES",
                     help="instead of the default workload: prefill / decode throughput of the ragged-step engine's latent-attention + "
                          "state-space model beside the dense Llama-shaped stack of equal width; comma-separated sizes of " + ", ".join(SEQ_BENCH_SIZES))
@@ -842,6 +906,8 @@ def main():
         return bench_gutivik(args, dev)
     if args.gaparax:
         return bench_gaparax(args, dev)
+    if args.zasazen:
+        return bench_zasazen(args, dev)
     from zhilight_amd import ops  # noqa: F401  (raises if the HIP library is missing)
     from zhilight_amd.llama import LLaMA, ModelConfig, QuantConfig
 

@@ -44,9 +44,10 @@ int zls_gemm_nt(const void* x, int64_t ldx, const void* w, void* y, int64_t ldy,
                 zl_stream_t s);
 /* The same product with an epilogue: y = act(x . w^T + bias), bias fp32 (n) nullable, act -1 none, 0 relu(v)^2, 1 gelu_tanh(v), 2 silu(v),
  * 3 softplus(v); y2 (nullable): the leading n2 columns of the result once more in `dtype` (rows of ldy2 >= n2 numbers) -- what a following
- * product reads while the rest of y stays fp32. */
+ * product reads while the rest of y stays fp32.  part (nullable): fp32 room for n_parts * m * n sums -- the tiled kernel then divides k over
+ * n_parts groups of workgroups (few output tiles, a long k), whose sums are added in order. */
 int zls_gemm_nt_act(const void* x, int64_t ldx, const void* w, const float* bias, int act, void* y, int64_t ldy, void* y2, int64_t ldy2, int64_t n2,
-                    int64_t m, int64_t n, int64_t k, int dtype, int out_dtype, zl_stream_t s);
+                    int64_t m, int64_t n, int64_t k, float* part, int64_t n_parts, int dtype, int out_dtype, zl_stream_t s);
 /* The same with gathered rows: row r of x is x[x_rows[r]], row c of w is w[w_rows[c]] (device int32 arrays, NULL: in order; ldw: row
  * stride of w).  Always the tiled kernel.  The up-projection of cached rows that lie scattered over pages. */
 int zls_gemm_nt_gather(const void* x, int64_t ldx, const int32_t* x_rows, const void* w, int64_t ldw, const int32_t* w_rows, void* y,

@@ -175,6 +175,21 @@ template <> struct VecF<4> {
     static __device__ __forceinline__ void st(float* p, const float* v) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
 };
 
+// V consecutive numbers in the serving format (V = 4: one access)
+template <int DT, int V>
+__device__ __forceinline__ void st_row(void* p, size_t at, const float* v) {
+    if constexpr (V == 4 && DT == ZL_BF16) {
+        uint32_t h[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) h[e] = ZT<ZL_BF16>::from_f32(v[e]);
+        *reinterpret_cast<uint2*>(reinterpret_cast<uint16_t*>(p) + at) = make_uint2(h[0] | h[1] << 16, h[2] | h[3] << 16);
+    } else if constexpr (V == 4) {
+        *reinterpret_cast<float4*>(reinterpret_cast<float*>(p) + at) = make_float4(v[0], v[1], v[2], v[3]);
+    } else {
+        SeqT<DT>::st(p, at, v[0]);
+    }
+}
+
 constexpr int kMaxBranches = 4;
 
 struct BranchP {
@@ -236,17 +251,21 @@ __global__ __launch_bounds__(kT) void k_add_branches(const BranchP p) {
         }
         VecF<V>::st(u + i, x);
 #pragma unroll
-        for (int e = 0; e < V; ++e) {
-            sx = fmaf(x[e], x[e], sx);
-            if (p.xt) SeqT<DT>::st(p.xt, (size_t)blockIdx.x * p.ldxt + i + e, x[e]);
-        }
+        for (int e = 0; e < V; ++e) sx = fmaf(x[e], x[e], sx);
+        if (p.xt) st_row<DT, V>(p.xt, (size_t)blockIdx.x * p.ldxt + i, x);
     }
     if (!p.w1 && !p.w2) return;
     const float fx = 1.0f / sqrtf(zl_block_sum(sx, red) / (float)p.width + p.eps);
-    for (int i = threadIdx.x; i < p.width; i += kT) {
-        const float v = u[i] * fx;
-        if (p.w1) SeqT<DT>::st(p.h1, row + i, v * p.w1[i]);
-        if (p.w2) SeqT<DT>::st(p.h2, row + i, v * p.w2[i]);
+#pragma unroll 2
+    for (int i = threadIdx.x * V; i < p.width; i += kT * V) {                // (a thread reads back its own elements)
+        float v[V], a[V], c[V];
+        VecF<V>::ld(u + i, v);
+        if (p.w1) VecF<V>::ld(p.w1 + i, a);
+        if (p.w2) VecF<V>::ld(p.w2 + i, c);
+#pragma unroll
+        for (int e = 0; e < V; ++e) { v[e] *= fx; a[e] *= v[e]; c[e] *= v[e]; }
+        if (p.w1) st_row<DT, V>(p.h1, row + i, a);
+        if (p.w2) st_row<DT, V>(p.h2, row + i, c);
     }
 }
 
@@ -463,7 +482,7 @@ extern "C" int zls_add_branches(float* x, const zls_branch_t* branches, int64_t 
     ZL_CHECK_ARG(n <= kMaxBranches && width * sizeof(float) <= 60 * 1024, ZL_ELIMIT);
     BranchP p = {};
     auto al = [](const void* q) { return ((uintptr_t)q & 15) == 0; };
-    bool vec = width % 4 == 0 && al(x);
+    bool vec = width % 4 == 0 && al(x) && al(w1) && al(w2) && al(h1) && al(h2) && al(xt) && (!xt || ldxt % 4 == 0);
     for (int i = 0; i < n; ++i) {
         ZL_CHECK_ARG(branches[i].y, ZL_EINVAL);
         p.y[i] = branches[i].y; p.w[i] = branches[i].w; p.coef[i] = branches[i].coef;

@@ -9,6 +9,7 @@
 //   k_seq_gemm  more rows (prompt portions, mixed steps): 128 x 128 or 64 x 64 output tile per workgroup of 4 waves (2 x 2; a wave =
 //               4 x 4 or 2 x 2 MFMA tiles of 16 x 16), 32-k slices of x and W staged through LDS (zero-filled past the edges), the next slice's global
 //               loads issued before the current slice's MFMAs.  bf16: v_mfma_f32_16x16x32_bf16; fp32: v_mfma_f32_16x16x4_f32.
+//               A long k with few output tiles is divided over workgroups (blockIdx.z), k_split_sum adds the parts.
 // Each has an instantiation with an epilogue (EPI: bias, activation, leading columns once more in the serving format).
 #include "seq_common.h"
 
@@ -34,6 +35,8 @@ struct GemmP {
     // columns once more in the format of x to y2 (nullable): what a following product reads while the rest stays fp32
     const float* bias; int uact;
     void* y2; int64_t ldy2; int n2;
+    // few output tiles and a long k: blockIdx.z takes k_part numbers of k and leaves its plain sums in part (parts, m, n); k_split_sum adds them
+    float* part; int k_part, n_parts;
 };
 
 template <int DT, int ODT, bool EPI>
@@ -109,6 +112,7 @@ __global__ __launch_bounds__(256) void k_seq_gemm(const GemmP p) {
         wbase = reinterpret_cast<const E*>(p.w) + (size_t)e * p.w_stride;
     }
     const int lrow = tid >> 2, lkc = (tid & 3) * 8;
+    const int kbeg = p.part ? blockIdx.z * p.k_part : 0, kend = p.part ? min(p.k, kbeg + p.k_part) : p.k;      // (k_part: whole slices)
 
     f4 acc[WT][WT];
 #pragma unroll
@@ -126,10 +130,10 @@ __global__ __launch_bounds__(256) void k_seq_gemm(const GemmP p) {
         wr[u] = (p.w_rows && nr < p.n) ? p.w_rows[nr] : nr;
         xlim[u] = mr < mlim ? xr[u] + 1 : 0;
         wlim[u] = nr < p.n ? wr[u] + 1 : 0;
-        tx[u].load(p.x, p.ldx, xr[u], xlim[u], 0, lkc, p.k, p.vec);
-        tw[u].load(wbase, p.ldw, wr[u], wlim[u], 0, lkc, p.k, p.vec);
+        tx[u].load(p.x, p.ldx, xr[u], xlim[u], kbeg, lkc, p.k, p.vec);
+        tw[u].load(wbase, p.ldw, wr[u], wlim[u], kbeg, lkc, p.k, p.vec);
     }
-    for (int k0 = 0; k0 < p.k; k0 += kBK) {
+    for (int k0 = kbeg; k0 < kend; k0 += kBK) {
         __syncthreads();                                        // the previous slice's fragments are consumed
 #pragma unroll
         for (int u = 0; u < PASS; ++u) {
@@ -137,7 +141,7 @@ __global__ __launch_bounds__(256) void k_seq_gemm(const GemmP p) {
             tw[u].store(ws, lrow + 64 * u, lkc);
         }
         __syncthreads();
-        if (k0 + kBK < p.k) {                                   // next slice in flight during the MFMAs
+        if (k0 + kBK < kend) {                                  // next slice in flight during the MFMAs
 #pragma unroll
             for (int u = 0; u < PASS; ++u) {
                 tx[u].load(p.x, p.ldx, xr[u], xlim[u], k0 + kBK, lkc, p.k, p.vec);
@@ -195,9 +199,22 @@ __global__ __launch_bounds__(256) void k_seq_gemm(const GemmP p) {
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int row = m0 + wm * 16 * WT + i * 16 + 4 * kq + r;
-                if (row < mlim && col < p.n) put<DT, ODT, EPI>(p, row, col, acc[i][j][r]);
+                if (row < mlim && col < p.n) {
+                    if (p.part) p.part[((size_t)blockIdx.z * p.m + row) * p.n + col] = acc[i][j][r];
+                    else put<DT, ODT, EPI>(p, row, col, acc[i][j][r]);
+                }
             }
         }
+}
+
+// the parts of a k that was divided, added in order, and the epilogue
+template <int DT, int ODT, bool EPI>
+__global__ __launch_bounds__(256) void k_split_sum(const GemmP p) {
+    const int64_t e = (int64_t)blockIdx.x * 256 + threadIdx.x, mn = (int64_t)p.m * p.n;
+    if (e >= mn) return;
+    float v = 0.f;
+    for (int z = 0; z < p.n_parts; ++z) v += p.part[z * mn + e];
+    put<DT, ODT, EPI>(p, (int)(e / p.n), (int)(e % p.n), v);
 }
 
 // ---- a few rows: the weights are the traffic -----------------------------------------------------------------------------------------
@@ -357,7 +374,11 @@ __global__ __launch_bounds__(256) void k_seq_gemv_grouped(const GemmP p, const i
 template <int DT, int ODT, bool EPI = false>
 void launch_tiled(const GemmP& p, hipStream_t hs) {
     const int64_t big = (int64_t)((p.m + 127) / 128) * ((p.n + 127) / 128);
-    if (big >= 256) {
+    if (p.part) {
+        const dim3 grid((unsigned)((p.n + 63) / 64), (unsigned)((p.m + 63) / 64), (unsigned)p.n_parts);
+        hipLaunchKernelGGL((k_seq_gemm<DT, ODT, 2, false, EPI>), grid, dim3(256), 0, hs, p);
+        hipLaunchKernelGGL((k_split_sum<DT, ODT, EPI>), dim3((unsigned)(((int64_t)p.m * p.n + 255) / 256)), dim3(256), 0, hs, p);
+    } else if (big >= 256) {
         const dim3 grid((unsigned)((p.n + 127) / 128), (unsigned)((p.m + 127) / 128));
         hipLaunchKernelGGL((k_seq_gemm<DT, ODT, 4, false, EPI>), grid, dim3(256), 0, hs, p);
     } else {
@@ -369,12 +390,12 @@ void launch_tiled(const GemmP& p, hipStream_t hs) {
 template <int DT, int ODT, bool EPI = false>
 int launch(const GemmP& p, hipStream_t hs) {
     if constexpr (DT == ZL_BF16) {
-        if (p.m >= 3 && p.m <= 16 && p.vec && (p.k & 7) == 0) {
+        if (!p.part && p.m >= 3 && p.m <= 16 && p.vec && (p.k & 7) == 0) {
             hipLaunchKernelGGL((k_seq_gemv_mfma<ODT, EPI>), dim3((unsigned)((p.n + 15) / 16)), dim3(256), 0, hs, p);
             return zl_launch_status();
         }
     }
-    if (p.m <= 8) {
+    if (p.m <= 8 && !p.part) {
         if (p.m <= 2) hipLaunchKernelGGL((k_seq_gemv<DT, ODT, 2, 1, EPI>), dim3((unsigned)((p.n + 3) / 4)), dim3(256), 0, hs, p);
         else if (p.m <= 4) hipLaunchKernelGGL((k_seq_gemv<DT, ODT, 4, 2, EPI>), dim3((unsigned)((p.n + 7) / 8)), dim3(256), 0, hs, p);
         else hipLaunchKernelGGL((k_seq_gemv<DT, ODT, 8, 4, EPI>), dim3((unsigned)((p.n + 15) / 16)), dim3(256), 0, hs, p);
@@ -389,7 +410,7 @@ int launch(const GemmP& p, hipStream_t hs) {
 extern "C" int zls_version(void) { return 1; }
 
 extern "C" int zls_gemm_nt_act(const void* x, int64_t ldx, const void* w, const float* bias, int act, void* y, int64_t ldy, void* y2, int64_t ldy2,
-                               int64_t n2, int64_t m, int64_t n, int64_t k, int dtype, int out_dtype, zl_stream_t s) {
+                               int64_t n2, int64_t m, int64_t n, int64_t k, float* part, int64_t n_parts, int dtype, int out_dtype, zl_stream_t s) {
     ZL_CHECK_ARG(x && w && y && m > 0 && n > 0 && k > 0, ZL_EINVAL);
     ZL_CHECK_ARG(ldx >= k && ldy >= n && m < (1 << 30) && n < (1 << 30) && k < (1 << 30), ZL_ESHAPE);
     ZL_CHECK_ARG((m + 63) / 64 <= 65535, ZL_ELIMIT);
@@ -399,6 +420,12 @@ extern "C" int zls_gemm_nt_act(const void* x, int64_t ldx, const void* w, const 
     GemmP p = {};
     p.x = x; p.w = w; p.y = y; p.ldx = ldx; p.ldw = k; p.ldy = ldy; p.m = (int)m; p.n = (int)n; p.k = (int)k;
     p.x_rows = p.w_rows = nullptr; p.tiles = nullptr; p.w_stride = 0;
+    if (part) {
+        ZL_CHECK_ARG(n_parts > 0 && n_parts <= 65535, ZL_EINVAL);
+        p.k_part = (int)((k + n_parts * kBK - 1) / (n_parts * kBK) * kBK);
+        p.n_parts = (int)((k + p.k_part - 1) / p.k_part);                // (never more than the caller made room for)
+        p.part = part;
+    }
     p.bias = bias; p.uact = act; p.y2 = y2; p.ldy2 = ldy2; p.n2 = y2 ? (int)n2 : 0;
     const int64_t unit = dtype == ZL_BF16 ? 8 : 4;
     p.vec = (k % unit == 0 && ldx % unit == 0 && ((uintptr_t)x & 15) == 0 && ((uintptr_t)w & 15) == 0) ? 1 : 0;
@@ -413,7 +440,7 @@ extern "C" int zls_gemm_nt_act(const void* x, int64_t ldx, const void* w, const 
 
 extern "C" int zls_gemm_nt(const void* x, int64_t ldx, const void* w, void* y, int64_t ldy, int64_t m, int64_t n, int64_t k, int dtype,
                            int out_dtype, zl_stream_t s) {
-    return zls_gemm_nt_act(x, ldx, w, nullptr, -1, y, ldy, nullptr, 0, 0, m, n, k, dtype, out_dtype, s);
+    return zls_gemm_nt_act(x, ldx, w, nullptr, -1, y, ldy, nullptr, 0, 0, m, n, k, nullptr, 0, dtype, out_dtype, s);
 }
 
 // the same product with GATHERED rows of x and / or w (x_rows / w_rows: device int32 row indices, NULL: the rows in order), always on the

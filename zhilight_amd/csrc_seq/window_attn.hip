@@ -6,8 +6,8 @@
 // bias by the distance between query and key, queries confined to their chunk of positions, and weights that are sigmoids instead of a
 // softmax (every key on its own; the splits of a token are then plain sums).
 //
-// k_rope_norm_store    a workgroup per token, a wave per head in turn: the head's coordinates in registers, rotated, normed, written back
-//                      (queries, fp32, in place) or to the token's row of the paged planes (keys, values; serving format)
+// k_rope_norm_store    workgroups per token for queries, for keys and values, and for another mixer's heads out of the same row; a wave per head
+//                      in turn: the head's coordinates in registers, rotated, normed, written back (queries, fp32, in place) or to the token's row of the paged planes (keys, values; serving format)
 // k_window_attention   a workgroup per (token, query head, split of the window's pages): a page of keys at a time -- a wave per key for the
 //                      scores (butterfly over the head size), running maximum and sum, then a thread per output coordinate for P.V over the
 //                      page's transposed values.  Single decoded tokens in both formats, and everything in fp32.
@@ -26,11 +26,26 @@ constexpr int kMaxE = 8;            // coordinates of a head per lane: dim, vdim
 constexpr int kChunk = 128;         // the largest page k_window_attention walks
 constexpr int kMaxV = 8;            // output coordinates per thread: (all_kv ? kv_heads : 1) * vdim <= 256 * kMaxV
 
-// one head of `size` coordinates in the lanes' registers (coordinate i in lane i % 64, register i / 64): rotate the first n_rot (pairs
-// i, i + n_rot / 2; interleaved: pairs 2i, 2i + 1) by pos * freq[i], optionally divide by the root mean square; the result stays in v[].
-// pre / pre_w: a factor and a weight per coordinate that the numbers get before anything else
-__device__ __forceinline__ void rope_head(float* v, const float* src, int size, int n_rot, const float* __restrict__ freq, float pos, bool norm,
-                                          float eps, int lane, bool interleaved = false, const float* __restrict__ w = nullptr, float pre = 1.0f,
+// The sines and cosines that a wave's lanes need for the rotated coordinates of any head (coordinate i in lane i % 64, register i / 64):
+// worked out once per token, used by all its heads
+struct Turn {
+    float sn[kMaxE], cs[kMaxE];
+    __device__ __forceinline__ void set(int n_rot, const float* __restrict__ freq, float pos, int lane, bool interleaved) {
+        const int half = n_rot >> 1;
+#pragma unroll
+        for (int r = 0; r < kMaxE; ++r) {
+            const int i = lane + 64 * r;
+            sn[r] = 0.f; cs[r] = 1.f;
+            if (i < n_rot) seq_sincos(pos * freq[interleaved ? (i >> 1) : (i < half ? i : i - half)], &sn[r], &cs[r]);
+        }
+    }
+};
+
+// one head of `size` coordinates in the lanes' registers: rotate the first n_rot (pairs i, i + n_rot / 2; interleaved: pairs 2i, 2i + 1),
+// optionally divide by the root mean square; the result stays in v[].  pre / pre_w: a factor and a weight per coordinate that the numbers get
+// before anything else
+__device__ __forceinline__ void rope_head(float* v, const float* src, int size, int n_rot, const Turn& turn, bool norm, float eps, int lane,
+                                          bool interleaved = false, const float* __restrict__ w = nullptr, float pre = 1.0f,
                                           const float* __restrict__ pre_w = nullptr) {
     const int half = n_rot >> 1;
     float ss = 0.f;
@@ -44,9 +59,7 @@ __device__ __forceinline__ void rope_head(float* v, const float* src, int size, 
                 const bool lo = interleaved ? (i & 1) == 0 : i < half;
                 const int oi = interleaved ? (i ^ 1) : (lo ? i + half : i - half);
                 const float other = pre_w ? src[oi] * pre * pre_w[oi] : src[oi] * pre;
-                float sn, cs;
-                seq_sincos(pos * freq[interleaved ? (i >> 1) : (lo ? i : i - half)], &sn, &cs);
-                o = lo ? o * cs - other * sn : o * cs + other * sn;
+                o = lo ? o * turn.cs[r] - other * turn.sn[r] : o * turn.cs[r] + other * turn.sn[r];
             }
             ss = fmaf(o, o, ss);
         }
@@ -71,67 +84,75 @@ struct RopeP {
     zls_head_prep_t prep;                           // norms over whole rows, query temperature, further heads (all zero: none)
 };
 
+// The workgroups of a token (blockIdx.y): 0 the queries, 1 keys and values, 2 .. the further heads.  A token's queries stay in one workgroup: with a norm
+// over all of them it has to read the whole row before it writes any of it
 template <int DT>
 __global__ __launch_bounds__(256) void k_rope_norm_store(const RopeP p, const zls_batch_t b) {
+    __shared__ float red[16];
     const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int sq = b.tok_seq[t];
     const int posi = b.seq_pos0[sq] + (t - b.seq_start[sq]);
     const float pos = (float)posi;
     float* row = p.proj + (size_t)t * p.ld;
-    const size_t cpage = (size_t)b.page_table[(size_t)sq * b.max_pages + posi / b.page_size];
-    const size_t crow = cpage * b.page_size + posi % b.page_size;
-    const int n_kv = p.k_cache ? p.kv_heads : 0;
-    float fq = 1.0f, fk = 1.0f, temp = 1.0f;
-    if (p.prep.whole_norm) {                                             // one root mean square over all query heads, one over all key heads
-        __shared__ float red[16];
-        const int nq = p.heads * p.dim, nk = n_kv * p.dim;
-        float sq_ = 0.f, sk_ = 0.f;
-        for (int i = threadIdx.x; i < nq; i += 256) { const float u = row[p.q_col0 + i]; sq_ = fmaf(u, u, sq_); }
-        for (int i = threadIdx.x; i < nk; i += 256) { const float u = row[p.k_col0 + i]; sk_ = fmaf(u, u, sk_); }
-        fq = 1.0f / sqrtf(zl_block_sum(sq_, red) / (float)nq + p.eps);   // (its barriers: every wave has read the row before one writes it)
-        if (nk) fk = 1.0f / sqrtf(zl_block_sum(sk_, red) / (float)nk + p.eps);
-    }
-    if (p.prep.temp_every > 0) temp = 1.0f + p.prep.temp_coef * logf((float)((posi + 1) / p.prep.temp_every + 1));
+    Turn turn;
     float v[kMaxE];
-    for (int h = wave; h < p.heads + 2 * n_kv + p.prep.x_heads; h += 4) {          // (a wave owns its heads: no two waves touch the same numbers)
-        if (h >= p.heads + 2 * n_kv) {
-            float* x = row + p.prep.x_col0 + (h - p.heads - 2 * n_kv) * p.prep.x_dim;
-            rope_head(v, x, p.prep.x_dim, p.prep.x_rot, p.prep.x_freq, pos, false, 0.f, lane);
+    if (blockIdx.y >= 2) {
+        turn.set(p.prep.x_rot, p.prep.x_freq, pos, lane, false);
+        for (int h = (blockIdx.y - 2) * 4 + wave; h < p.prep.x_heads; h += (gridDim.y - 2) * 4) {      // (a wave owns its heads)
+            float* x = row + p.prep.x_col0 + h * p.prep.x_dim;
+            rope_head(v, x, p.prep.x_dim, p.prep.x_rot, turn, false, 0.f, lane);
 #pragma unroll
             for (int r = 0; r < kMaxE; ++r)
                 if (lane + 64 * r < p.prep.x_rot) x[lane + 64 * r] = v[r];
-        } else if (h < p.heads) {
-            float* q = row + p.q_col0 + h * p.dim;
-            rope_head(v, q, p.dim, p.rot_dims, p.qk_freq, pos, p.qk_norm != 0, p.eps, lane, p.interleaved != 0, p.q_w, fq,
-                      p.prep.q_w ? p.prep.q_w + h * p.dim : nullptr);
-            if (p.prep.temp_every > 0) {
-#pragma unroll
-                for (int r = 0; r < kMaxE; ++r) v[r] *= temp;
-            }
-#pragma unroll
-            for (int r = 0; r < kMaxE; ++r)
-                if (lane + 64 * r < p.dim) q[lane + 64 * r] = v[r];
-        } else if (h < p.heads + n_kv) {
-            const int c = h - p.heads;
-            rope_head(v, row + p.k_col0 + c * p.dim, p.dim, p.rot_dims, p.qk_freq, pos, p.qk_norm != 0, p.eps, lane, p.interleaved != 0, p.k_w, fk,
-                      p.prep.k_w ? p.prep.k_w + c * p.dim : nullptr);
-#pragma unroll
-            for (int r = 0; r < kMaxE; ++r)
-                if (lane + 64 * r < p.dim) SeqT<DT>::st(p.k_cache, (crow * p.kv_heads + c) * p.dim + lane + 64 * r, v[r]);
-        } else {
-            const int c = h - p.heads - n_kv;
-            rope_head(v, row + p.v_col0 + c * p.vdim, p.vdim, p.v_freq ? p.vdim : 0, p.v_freq, pos, false, 0.f, lane);
-            if (p.vmix_src) {
-                const float* other = p.vmix_src + (size_t)t * p.vmix_ld + p.vmix_col0 + c * p.vdim;
-#pragma unroll
-                for (int r = 0; r < kMaxE; ++r)
-                    if (lane + 64 * r < p.vdim) v[r] = (1.0f - p.vmix_lambda) * v[r] + p.vmix_lambda * other[lane + 64 * r];
-            }
-#pragma unroll
-            for (int r = 0; r < kMaxE; ++r)
-                if (lane + 64 * r < p.vdim)                             // values lie transposed inside a page: (kv head, coordinate, key)
-                    SeqT<DT>::st(p.v_cache, ((cpage * p.kv_heads + c) * p.vdim + lane + 64 * r) * b.page_size + posi % b.page_size, v[r]);
         }
+        return;
+    }
+    const bool queries = blockIdx.y == 0;
+    if (!queries && !p.k_cache) return;                                  // (a layer that only reads another one's cache)
+    float f = 1.0f;
+    if (p.prep.whole_norm) {                                             // one root mean square over all query heads, one over all key heads
+        const float* src = row + (queries ? p.q_col0 : p.k_col0);
+        const int n = (queries ? p.heads : p.kv_heads) * p.dim;
+        float ss = 0.f;
+        for (int i = threadIdx.x; i < n; i += 256) { const float u = src[i]; ss = fmaf(u, u, ss); }
+        f = 1.0f / sqrtf(zl_block_sum(ss, red) / (float)n + p.eps);      // (its barriers: every wave has read the row before one writes it)
+    }
+    turn.set(p.rot_dims, p.qk_freq, pos, lane, p.interleaved != 0);
+    if (queries) {
+        const float temp = p.prep.temp_every > 0 ? 1.0f + p.prep.temp_coef * logf((float)((posi + 1) / p.prep.temp_every + 1)) : 1.0f;
+        for (int h = wave; h < p.heads; h += 4) {                        // (a wave owns its heads: no two waves touch the same numbers)
+            float* q = row + p.q_col0 + h * p.dim;
+            rope_head(v, q, p.dim, p.rot_dims, turn, p.qk_norm != 0, p.eps, lane, p.interleaved != 0, p.q_w, f,
+                      p.prep.q_w ? p.prep.q_w + h * p.dim : nullptr);
+#pragma unroll
+            for (int r = 0; r < kMaxE; ++r)
+                if (lane + 64 * r < p.dim) q[lane + 64 * r] = v[r] * temp;
+        }
+        return;
+    }
+    const size_t cpage = (size_t)b.page_table[(size_t)sq * b.max_pages + posi / b.page_size];
+    const size_t crow = cpage * b.page_size + posi % b.page_size;
+    for (int c = wave; c < p.kv_heads; c += 4) {
+        rope_head(v, row + p.k_col0 + c * p.dim, p.dim, p.rot_dims, turn, p.qk_norm != 0, p.eps, lane, p.interleaved != 0, p.k_w, f,
+                  p.prep.k_w ? p.prep.k_w + c * p.dim : nullptr);
+#pragma unroll
+        for (int r = 0; r < kMaxE; ++r)
+            if (lane + 64 * r < p.dim) SeqT<DT>::st(p.k_cache, (crow * p.kv_heads + c) * p.dim + lane + 64 * r, v[r]);
+    }
+    const int v_rot = p.v_freq ? p.vdim : 0;
+    turn.set(v_rot, p.v_freq, pos, lane, false);
+    for (int c = wave; c < p.kv_heads; c += 4) {
+        rope_head(v, row + p.v_col0 + c * p.vdim, p.vdim, v_rot, turn, false, 0.f, lane);
+        if (p.vmix_src) {
+            const float* other = p.vmix_src + (size_t)t * p.vmix_ld + p.vmix_col0 + c * p.vdim;
+#pragma unroll
+            for (int r = 0; r < kMaxE; ++r)
+                if (lane + 64 * r < p.vdim) v[r] = (1.0f - p.vmix_lambda) * v[r] + p.vmix_lambda * other[lane + 64 * r];
+        }
+#pragma unroll
+        for (int r = 0; r < kMaxE; ++r)
+            if (lane + 64 * r < p.vdim)                                 // values lie transposed inside a page: (kv head, coordinate, key)
+                SeqT<DT>::st(p.v_cache, ((cpage * p.kv_heads + c) * p.vdim + lane + 64 * r) * b.page_size + posi % b.page_size, v[r]);
     }
 }
 
@@ -706,8 +727,10 @@ extern "C" int zls_rope_norm_store(float* proj, int64_t ld, int64_t q_col0, int6
     p.v_freq = v_freq; p.eps = eps; p.k_cache = k_cache; p.v_cache = v_cache;
     ZL_CHECK_ARG(!vmix_src || (vmix_col0 >= 0 && vmix_col0 + kv_heads * vdim <= vmix_ld), ZL_ESHAPE);
     p.q_w = qk_norm ? q_norm_w : nullptr; p.k_w = qk_norm ? k_norm_w : nullptr;
+    const int extra = (p.prep.x_heads + 3) / 4;                          // four further heads per workgroup, a few workgroups when tokens are many
+    const unsigned parts = extra ? 2u + (unsigned)(extra > 4 && b->n_tok > 64 ? 4 : extra > 64 ? 64 : extra) : k_cache ? 2u : 1u;
     p.interleaved = interleaved ? 1 : 0; p.vmix_src = vmix_src; p.vmix_ld = vmix_ld; p.vmix_col0 = (int)vmix_col0; p.vmix_lambda = vmix_lambda;
-#define CALL(DT) hipLaunchKernelGGL((k_rope_norm_store<DT>), dim3(b->n_tok), dim3(256), 0, (hipStream_t)s, p, *b);
+#define CALL(DT) hipLaunchKernelGGL((k_rope_norm_store<DT>), dim3(b->n_tok, parts), dim3(256), 0, (hipStream_t)s, p, *b);
     ZLS_DISPATCH(dtype, CALL)
 #undef CALL
     return zl_launch_status();

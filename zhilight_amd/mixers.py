@@ -169,7 +169,7 @@ class Mamba2Mixer:
         self.taps, self.norm_groups, self.eps = taps, norm_groups, float(eps)
         self.inner = heads * vdim
         self.channels = self.inner + 2 * groups * n_state
-        self.scan_segment = None          # tokens per segment of a long portion (None: seqops.SCAN_SEGMENT; 0: never in segments)
+        self.scan_segment = None          # tokens per segment of a long portion (None: seqops.scan_segment; 0: never in segments)
 
     def load(self, get, prefix, dtype, device):
         W = self.width
@@ -622,7 +622,7 @@ class Mamba1Mixer:
             raise ZLError("mamba1: sizes must be positive")
         self.name, self.width, self.inner, self.n_state, self.rank, self.taps = name, width, inner, n_state, rank, taps
         self.low = (rank + 7) // 8 * 8
-        self.scan_segment = None          # tokens per segment of a long portion (None: seqops.SELECTIVE_SEGMENT; 0: never in segments)
+        self.scan_segment = None          # tokens per segment of a long portion (None: seqops.scan_segment; 0: never in segments)
 
     def _pack(self, w_x, w_dt, a_log):
         r, low = self.rank, self.low

@@ -185,6 +185,14 @@ class RaggedBatch:
         return self._windowed[window]
 
 
+def _k_parts(m, n, k):
+    """over how many workgroups per output tile a product divides k: a tiled product whose tiles leave most of the chip idle"""
+    if m <= 16 or k < 512:
+        return 1
+    tiles = ((m + 63) // 64) * ((n + 63) // 64)
+    return 1 if tiles > 128 else max(1, min(256 // tiles, k // 256, 16))
+
+
 def gemm_nt(x, w, out=None, out_dtype=torch.float32, bias=None, act=None, lead=0):
     """act(x (m, k) . w (n, k)^T + bias) -> (m, n); x and w in the serving format, the result fp32 (or that format); bias fp32 (n) or None,
     act one of UNARY_ACTS or None.  lead > 0: returns (result, its leading `lead` columns once more in the serving format)"""
@@ -203,8 +211,10 @@ def gemm_nt(x, w, out=None, out_dtype=torch.float32, bias=None, act=None, lead=0
     elif out.shape != (m, n) or not out.is_contiguous():
         raise ZLError("gemm_nt: wrong output")
     y2 = torch.empty((m, lead), dtype=x.dtype, device=x.device) if lead > 0 else None
+    parts = _k_parts(m, n, k)
+    part = torch.empty((parts, m, n), dtype=torch.float32, device=x.device) if parts > 1 else None
     check(lib().zls_gemm_nt_act(_p(x), _i(x.stride(0)), _p(w), _p(bias), C.c_int(-1 if act is None else UNARY_ACTS[act]), _p(out), _i(n), _p(y2),
-                                _i(lead), _i(lead), _i(m), _i(n), _i(k), C.c_int(dt_code(x.dtype)), C.c_int(dt_code(out.dtype)), _stream()), "gemm_nt")
+                                _i(lead), _i(lead), _i(m), _i(n), _i(k), _p(part), _i(parts), C.c_int(dt_code(x.dtype)), C.c_int(dt_code(out.dtype)), _stream()), "gemm_nt")
     return (out, y2) if lead > 0 else out
 
 
@@ -354,7 +364,21 @@ def short_conv(proj, col0, w, in_bias, tail, batch, act=False, bias=None, also=N
     return out if also is None else (out, out if out_t is None else out_t)
 
 
-SCAN_SEGMENT = 256      # tokens per segment of a long portion (ssm_scan)
+SCAN_SEGMENT = 256      # tokens per segment of a long portion, at most (ssm_scan, decay_scan)
+SCAN_WAVES = 2048       # waves that a scan of one step should bring onto the chip
+
+
+def scan_segment(n_tok, waves, longest, shortest=16):
+    """tokens per segment for a scan that runs `waves` waves per segment: as long as the step's segments together still make SCAN_WAVES waves"""
+    return max(shortest, min(longest, (n_tok * waves // SCAN_WAVES + 15) // 16 * 16))
+
+
+def _scan_waves(heads, columns, n_state):
+    """waves of one segment of the scan kernel: per head a thread for every value column and group of at most 32 states"""
+    lanes = 1
+    while (n_state + lanes - 1) // lanes > 32:
+        lanes *= 2
+    return heads * ((lanes * columns + 63) // 64)
 
 
 def ssm_scan(xbc, proj, dt_col0, dt_bias, a_log, d, state, heads, vdim, n_state, groups, batch, seg_len=None):
@@ -363,7 +387,7 @@ def ssm_scan(xbc, proj, dt_col0, dt_bias, a_log, d, state, heads, vdim, n_state,
     if xbc.shape[1] != heads * vdim + 2 * groups * n_state or tuple(state.shape[1:]) != (heads, n_state, vdim):
         raise ZLError("ssm_scan: shapes")
     y = torch.empty((batch.n_tok, heads * vdim), dtype=torch.float32, device=xbc.device)
-    seg_len = SCAN_SEGMENT if seg_len is None else seg_len
+    seg_len = scan_segment(batch.n_tok, _scan_waves(heads, vdim, n_state), SCAN_SEGMENT) if seg_len is None else seg_len
     ws = None
     if seg_len > 0 and batch.c.max_count > seg_len:
         ws = torch.empty(int(lib().zls_ssm_scan_workspace_bytes(_i(batch.n_seq), _i(batch.c.max_count), _i(seg_len), _i(heads), _i(vdim),
@@ -373,7 +397,7 @@ def ssm_scan(xbc, proj, dt_col0, dt_bias, a_log, d, state, heads, vdim, n_state,
     return y
 
 
-SELECTIVE_SEGMENT = 128     # tokens per segment of a long portion (selective_scan)
+SELECTIVE_SEGMENT = 128     # tokens per segment of a long portion, at most (selective_scan)
 
 
 def selective_scan(x, dt, bc, b_col0, c_col0, zrow, z_col0, a2, d, state, batch, dtype, seg_len=None):
@@ -386,7 +410,8 @@ def selective_scan(x, dt, bc, b_col0, c_col0, zrow, z_col0, a2, d, state, batch,
             n_tok != batch.n_tok or bc.shape[0] != n_tok or zrow.shape[0] != n_tok:
         raise ZLError("selective_scan: shapes")
     y = torch.empty((n_tok, inner), dtype=dtype, device=x.device)
-    seg_len = SELECTIVE_SEGMENT if seg_len is None else seg_len
+    if seg_len is None:
+        seg_len = scan_segment(batch.n_tok, (inner + 63) // 64 * ((n_state + 7) // 8), SELECTIVE_SEGMENT, 32)
     ws = None
     if seg_len > 0 and batch.c.max_count > seg_len:
         ws = torch.empty(int(lib().zls_selective_scan_workspace_bytes(_i(batch.n_seq), _i(batch.c.max_count), _i(seg_len), _i(inner), _i(n_state))) // 4,
@@ -682,7 +707,7 @@ def decay_scan(proj, q_col0, k_col0, v_col0, act, decay_h, decay_t, gain_t, norm
         if t is not None and tuple(t.shape) != (batch.n_tok, heads):
             raise ZLError("decay_scan: per-token decays / gains are (n_tok, heads)")
     y = torch.empty((batch.n_tok, heads * P), dtype=torch.float32, device=proj.device)
-    seg_len = SCAN_SEGMENT if seg_len is None else seg_len
+    seg_len = scan_segment(batch.n_tok, _scan_waves(heads, P, dim), SCAN_SEGMENT) if seg_len is None else seg_len
     ws = None
     if seg_len > 0 and batch.c.max_count > seg_len:
         ws = torch.empty(int(lib().zls_ssm_scan_workspace_bytes(_i(batch.n_seq), _i(batch.c.max_count), _i(seg_len), _i(heads), _i(P), _i(dim))) // 4,
