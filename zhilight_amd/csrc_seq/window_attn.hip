@@ -728,7 +728,8 @@ extern "C" int zls_rope_norm_store(float* proj, int64_t ld, int64_t q_col0, int6
     ZL_CHECK_ARG(!vmix_src || (vmix_col0 >= 0 && vmix_col0 + kv_heads * vdim <= vmix_ld), ZL_ESHAPE);
     p.q_w = qk_norm ? q_norm_w : nullptr; p.k_w = qk_norm ? k_norm_w : nullptr;
     const int extra = (p.prep.x_heads + 3) / 4;                          // four further heads per workgroup, a few workgroups when tokens are many
-    const unsigned parts = extra ? 2u + (unsigned)(extra > 4 && b->n_tok > 64 ? 4 : extra > 64 ? 64 : extra) : k_cache ? 2u : 1u;
+    const int most = b->n_tok > 512 ? 1 : b->n_tok > 64 ? 4 : 64;
+    const unsigned parts = extra ? 2u + (unsigned)(extra < most ? extra : most) : k_cache ? 2u : 1u;
     p.interleaved = interleaved ? 1 : 0; p.vmix_src = vmix_src; p.vmix_ld = vmix_ld; p.vmix_col0 = (int)vmix_col0; p.vmix_lambda = vmix_lambda;
 #define CALL(DT) hipLaunchKernelGGL((k_rope_norm_store<DT>), dim3(b->n_tok, parts), dim3(256), 0, (hipStream_t)s, p, *b);
     ZLS_DISPATCH(dtype, CALL)
