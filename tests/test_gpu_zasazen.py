@@ -182,7 +182,7 @@ def test_product_epilogues(dev, dtype, m):
     """bias, activation and the leading columns in the serving format, on every product kernel (few rows, up to 16, tiles)"""
     from zhilight_amd import seqops
     acts = {None: lambda z: z, "relu2": lambda z: torch.relu(z) ** 2, "gelu_tanh": O.gelu_tanh, "silu": O.silu, "softplus": O.softplus}
-    for n, k in ((70, 48), (200, 33)):
+    for n, k in ((70, 48), (200, 33), (40, 1000)):                              # (the last: k divided over workgroups above 16 rows)
         g = torch.Generator().manual_seed(n + m)
         x, w, b = bf(torch.randn(m, k, generator=g)), bf(torch.randn(n, k, generator=g) * 2 * k ** -0.5), torch.randn(n, generator=g)
         xd, wd, bd = x.to(dev).to(dtype), w.to(dev).to(dtype), b.to(dev)

@@ -222,8 +222,26 @@ __global__ __launch_bounds__(kT) void k_add_branches(const BranchP p) {
                     for (int e = 0; e < V; ++e) ss[b] = fmaf(v[e], v[e], ss[b]);
                 }
     float f[NB > 0 ? NB : 1];
+    if (any) {                                                               // all branches' sums behind one barrier: lanes, then waves in order
+        constexpr int W = kT / 64;
+        static_assert(kMaxBranches * W <= 16, "red holds a number per branch and wave");
 #pragma unroll
-    for (int b = 0; b < NB; ++b) f[b] = p.w[b] ? p.coef[b] / sqrtf(zl_block_sum(ss[b], red) / (float)p.width + p.eps) : p.coef[b];
+        for (int b = 0; b < NB; ++b) {
+            const float v = zl_wave_sum(ss[b]);
+            if ((threadIdx.x & 63) == 0) red[b * W + (threadIdx.x >> 6)] = v;
+        }
+        __syncthreads();
+    }
+#pragma unroll
+    for (int b = 0; b < NB; ++b) {
+        f[b] = p.coef[b];
+        if (p.w[b]) {
+            float t = 0.f;
+#pragma unroll
+            for (int w = 0; w < kT / 64; ++w) t += red[b * (kT / 64) + w];
+            f[b] = p.coef[b] / sqrtf(t / (float)p.width + p.eps);
+        }
+    }
     float sx = 0.f;
     for (int i = threadIdx.x * V; i < p.width; i += kT * V) {
         float x[V];

@@ -190,7 +190,7 @@ def _k_parts(m, n, k):
     if m <= 16 or k < 512:
         return 1
     tiles = ((m + 63) // 64) * ((n + 63) // 64)
-    return 1 if tiles > 128 else max(1, min(256 // tiles, k // 256, 16))
+    return 1 if tiles > 256 else max(1, min(512 // tiles, k // 256, 16))
 
 
 def gemm_nt(x, w, out=None, out_dtype=torch.float32, bias=None, act=None, lead=0):
