@@ -434,7 +434,7 @@ def test_retention_alone_in_portions_and_segments(dev, dtype, rh, rd, rv, rot):
     """rotated queries and keys, a fixed decay per head (one close to 1 with a far token that stands out), the norm per head"""
     from zhilight_amd.mixers import DecayLinearAttention
     W, T = 96, 230
-    layer = parallel_cfg(rh=rh, rd=rd, rv=rv, rot=rot, decay=[0.9990234375, 0.875, 0.96875, 1.0][:rh])
+    layer = parallel_cfg(rh=rh, rd=rd, rv=rv, rot=rot, decay=[0.998046875, 0.875, 0.984375, 1.0][:rh])
     m = layer["mixer"]["right"]
     sd = O.random_weights(model_cfg([layer], loop=None), 15, fixed_choice=True)
     h = bf(torch.randn(T, W, generator=torch.Generator().manual_seed(16)))
