@@ -45,9 +45,17 @@ int zls_gemm_nt(const void* x, int64_t ldx, const void* w, void* y, int64_t ldy,
 /* The same product with an epilogue: y = act(x . w^T + bias), bias fp32 (n) nullable, act -1 none, 0 relu(v)^2, 1 gelu_tanh(v), 2 silu(v),
  * 3 softplus(v); y2 (nullable): the leading n2 columns of the result once more in `dtype` (rows of ldy2 >= n2 numbers) -- what a following
  * product reads while the rest of y stays fp32.  part (nullable): fp32 room for n_parts * m * n sums -- the tiled kernel then divides k over
- * n_parts groups of workgroups (few output tiles, a long k), whose sums are added in order. */
+ * n_parts groups of workgroups (few output tiles, a long k), whose sums are added in order.
+ * factor (nullable): after the activation, result row r is multiplied by row rows[r] (clamped to 0 .. n_rows - 1) of a table in `dtype` --
+ * table points at the factor of column 0, rows are ld >= n numbers apart: a gate times an embedding looked up per token. */
+typedef struct {
+    const void* table;
+    const int32_t* rows;       /* device, (m) */
+    int64_t ld;
+    int32_t n_rows;
+} zls_row_factor_t;
 int zls_gemm_nt_act(const void* x, int64_t ldx, const void* w, const float* bias, int act, void* y, int64_t ldy, void* y2, int64_t ldy2, int64_t n2,
-                    int64_t m, int64_t n, int64_t k, float* part, int64_t n_parts, int dtype, int out_dtype, zl_stream_t s);
+                    const zls_row_factor_t* factor, int64_t m, int64_t n, int64_t k, float* part, int64_t n_parts, int dtype, int out_dtype, zl_stream_t s);
 /* The same with gathered rows: row r of x is x[x_rows[r]], row c of w is w[w_rows[c]] (device int32 arrays, NULL: in order; ldw: row
  * stride of w).  Always the tiled kernel.  The up-projection of cached rows that lie scattered over pages. */
 int zls_gemm_nt_gather(const void* x, int64_t ldx, const int32_t* x_rows, const void* w, int64_t ldw, const int32_t* w_rows, void* y,
@@ -188,7 +196,8 @@ int zls_add_layer_norm(float* x, const float* y, const float* w, const float* b,
  *   all kv_heads * dim key numbers by theirs, times q_w (heads * dim) / k_w (kv_heads * dim), fp32, nullable (qk_norm is 0 then);
  *   temp_every > 0: the finished queries are multiplied by 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1);
  *   x_heads > 0: x_heads more heads of x_dim numbers from column x_col0 of the same row are rotated in place, coordinate i < x_rot / 2 paired
- *   with i + x_rot / 2, angle p * x_freq[i] (fp32 (x_rot / 2)) -- another mixer's queries and keys out of the same projection. */
+ *   with i + x_rot / 2, angle p * x_freq[i] (fp32 (x_rot / 2)) -- another mixer's queries and keys out of the same projection;
+ *   rot_gain > 0: cos and sin of the queries' and keys' angles are multiplied by it (frequencies rescaled for long contexts). */
 typedef struct {
     int32_t whole_norm;
     const float* q_w;
@@ -197,6 +206,7 @@ typedef struct {
     int32_t temp_every;
     int32_t x_col0, x_heads, x_dim, x_rot;
     const float* x_freq;
+    float rot_gain;            /* factor on cos and sin of the queries and keys; 0: 1 */
 } zls_head_prep_t;
 
 /* Per token at position p, in place on the fp32 projection row proj[t] (ld floats):
@@ -263,10 +273,12 @@ int zls_window_attention_prompt(const float* q, int64_t ldq, int64_t q_col0, con
  * nullable: a learned score per head that has no key and no value and is not scaled; M then also covers it).
  * talk fp32 (heads, heads), NULL: no mixing, acc holds vdim numbers per head and split; v_freq (nullable): pair (m, m + vdim / 2) is turned
  * by -p * v_freq[m]; gate fp32 (n_tok, ldg) from g_col0, NULL: no gate; out (n_tok, heads * vdim) in `dtype`.
- * plain_sum != 0: the splits hold sums of finished weights (the sigmoid score form): a[t][g] = sum_s acc[t][g][s], no sink. */
+ * plain_sum != 0: the splits hold sums of finished weights (the sigmoid score form): a[t][g] = sum_s acc[t][g][s], no sink.
+ * gate_per_head != 0: the gate has ONE number per head, gate[t][g_col0 + h].  Rows of out have ldo >= heads * vdim numbers, every number is
+ * multiplied by out_scale before it is rounded. */
 int zls_head_mix_gate(const float* acc, const float* ml, int64_t n_splits, const float* talk, const float* v_freq, const float* gate,
                       int64_t ldg, int64_t g_col0, const float* sink, int plain_sum, const zls_batch_t* b, int64_t heads, int64_t kv_heads,
-                      int64_t vdim, void* out, int dtype, zl_stream_t s);
+                      int64_t vdim, int gate_per_head, float out_scale, void* out, int64_t ldo, int dtype, zl_stream_t s);
 
 /* ---- linear attention with a scalar decay per head and token ---------------------------------------------------------------------- */
 /* S_t = a_t S_{t-1} + b_t k_t v_t^T,  y_t = S_t^T q_t   per head, S fp32 (dim x vdim) carried in state[slot].
@@ -294,14 +306,33 @@ int zls_exp_gates(const float* proj, int64_t ld, int64_t i_col0, int64_t f_col0,
  *   with m_vals (needs norm_col): o = q_scale * o / (max(|q_scale * y[t][h][vdim]|, exp(-m_vals[t][h])) + den_eps);
  *   every one of `norm_groups` equal parts of the row heads * vdim is divided by sqrt(mean(part^2) + eps), times weight (nullable),
  *   times sigmoid(gate[t][g_col0 + c]) (gate nullable).  out (n_tok, heads * vdim) in `dtype`. */
-/* gate_kind 0: the gate is sigmoid(gate); 1: silu(gate).  Without m_vals o is only scaled by q_scale before the norm. */
+/* Rows of out have ldo >= heads * vdim numbers, every number is multiplied by out_scale before it is rounded.
+ * gate_kind 0: the gate is sigmoid(gate); 1: silu(gate).  Without m_vals o is only scaled by q_scale before the norm. */
 int zls_linear_attn_finish(const float* y, int64_t norm_col, float q_scale, const float* m_vals, float den_eps, int64_t heads, int64_t vdim,
                            int64_t norm_groups, const float* weight, float eps, const float* gate, int64_t ldg, int64_t g_col0,
-                           int64_t n_tok, void* out, int dtype, int gate_kind, zl_stream_t s);
+                           int64_t n_tok, float out_scale, void* out, int64_t ldo, int dtype, int gate_kind, zl_stream_t s);
 /* alpha[t][c] = sigmoid(sum_j w2[c][j] u[t][j] + bias[c])^(1 / tau) for c < channels: a decay per channel from `low` numbers per token,
  * u[t] = proj[t][u_col0 ..] fp32; w2 (channels, low) in `dtype`, bias fp32 (nullable); sums, the log-sigmoid and alpha are fp32. */
 int zls_lowrank_decay(const float* proj, int64_t ld, int64_t u_col0, int64_t low, const void* w2, const float* bias, float tau,
                       int64_t channels, int64_t n_tok, float* alpha, int dtype, zl_stream_t s);
+
+/* ---- gated delta rule --------------------------------------------------------------------------------------------------------------- */
+/* What a token needs before the recurrence.  Columns col0 .. of the fp32 rows proj[t] (ld) hold [q (kv_heads * dim) | k (kv_heads * dim) |
+ * v (heads * vdim)] = C channels: each passes a causal convolution (w fp32 (C, taps), last column: the current token; inputs before a
+ * portion from tail[slot] (taps - 1, C), which moves on; tail NULL when taps == 1) and SiLU; every q and k head is divided by
+ * sqrt(sum of its squares + unit_eps), q also multiplied by q_scale.  Results: qkv fp32 (n_tok, C); qk fp32 (n_tok, kv_heads) = q . k of the
+ * finished vectors; beta[t][h] = sigmoid(proj[t][b_col0 + h]); decay = exp(-rate[h] softplus(z + z_bias)) with z = z[t][z_col0 ..] (fp32
+ * rows of ldz), one number per head (per_channel 0, decay fp32 (n_tok, heads)) or per head and key channel (decay (n_tok, heads * dim));
+ * z_bias fp32, nullable, as many numbers.  dim <= 512. */
+int zls_delta_prep(const float* proj, int64_t ld, int64_t col0, const float* w, float* tail, int64_t taps, int64_t heads, int64_t kv_heads,
+                   int64_t dim, int64_t vdim, float q_scale, float unit_eps, int64_t b_col0, const float* z, int64_t ldz, int64_t z_col0,
+                   const float* z_bias, const float* rate, int per_channel, const zls_batch_t* b, float* qkv, float* qk, float* beta, float* decay,
+                   zl_stream_t s);
+/* Per head h (query / key head h / (heads / kv_heads)), tokens in order:  S <- g S (per key channel: row c of S by g[c]);
+ * u = beta (v - S^T k);  S <- S + k u^T;  y[t][h] = S^T q.  Inputs as zls_delta_prep left them.  state fp32 (slots, heads, vdim, dim) --
+ * the transpose of S, a value column's numbers side by side --, y fp32 (n_tok, heads * vdim).  dim <= 512. */
+int zls_delta_scan(const float* qkv, const float* qk, const float* beta, const float* decay, int per_channel, float* state, int64_t heads,
+                   int64_t kv_heads, int64_t dim, int64_t vdim, const zls_batch_t* b, float* y, zl_stream_t s);
 
 /* ---- mixture of experts over a ragged step ------------------------------------------------------------------------------------------ */
 /* Router: s = softmax(logits[t]) over all n_out outputs (score_kind 0), sigmoid(logits[t][i]) of each (score_kind 1) or logits[t] (score_kind
@@ -334,9 +365,10 @@ int zls_gemm_nt_grouped(const void* x, int64_t ldx, const int32_t* x_rows, const
 int zls_silu_mul(const float* gu, int64_t rows, int64_t ff, void* out, int dtype, zl_stream_t s);
 /* out[p][c] = act(g, u) of gu fp32 (rows, 2 ff) in `dtype`: kind 0 silu(g) u; 1 gelu_tanh(g) u (tanh form); 2 g' sigmoid(alpha g') (u' + 1)
  * with g' = min(g, limit), u' = clamp(u, -limit, limit).  block 0: g = gu[p][c], u = gu[p][ff + c]; block > 0 (ff % block == 0): the row
- * holds blocks of `block` gates followed by their `block` ups (the packing of the gated grouped product).  Rows of ld >= 2 ff numbers. */
-int zls_act_mul(const float* gu, int64_t ld, int64_t rows, int64_t ff, int kind, float alpha, float limit, int64_t block, void* out, int dtype,
-                zl_stream_t s);
+ * holds blocks of `block` gates followed by their `block` ups (the packing of the gated grouped product).  Rows of ld >= 2 ff numbers, out in
+ * rows of ldo >= ff. */
+int zls_act_mul(const float* gu, int64_t ld, int64_t rows, int64_t ff, int kind, float alpha, float limit, int64_t block, void* out, int64_t ldo,
+                int dtype, zl_stream_t s);
 /* out[t] = sum_k weights[t][k] * (ids[t][k] >= n_experts ? h[t] : y[slot_pos[t * top + k]]), in the order of k; y fp32 (.., width),
  * h (n_tok, width) in `dtype`, out fp32.  shared (nullable, fp32 (n_tok, width)): a shared expert's rows, added last, times
  * sigmoid(gate[t * ldg + g_col]) (gate nullable: times 1). */
@@ -349,6 +381,7 @@ int zls_moe_combine(const float* y, const int32_t* slot_pos, const int32_t* ids,
  *   x[t] += sum_i coef_i * (w_i ? y_i / sqrt(mean(y_i^2) + eps) * w_i : y_i)        in place, the sum in the order of the branches; n may be 0
  *   h1[t], h2[t] = x / sqrt(mean(x^2) + eps) * w1 | w2 of the NEW x in `dtype` (w1 / w2 nullable: two norms of one row share the mean)
  *   xt[t * ldxt ..] = the new x once more in `dtype` (nullable)
+ *   with tanh_b (nullable, fp32 (width); then w2 is NULL): h1[t] = tanh(tanh_alpha * x) * w1 + tanh_b instead, a norm without statistics
  * branches: host array; y, w, x fp32 device pointers.  width * 4 bytes <= 64 KiB. */
 typedef struct {
     const float* y;
@@ -356,7 +389,10 @@ typedef struct {
     float coef;
 } zls_branch_t;
 int zls_add_branches(float* x, const zls_branch_t* branches, int64_t n, float eps, int64_t rows, int64_t width, const float* w1, void* h1,
-                     const float* w2, void* h2, void* xt, int64_t ldxt, int dtype, zl_stream_t s);
+                     const float* w2, void* h2, void* xt, int64_t ldxt, const float* tanh_b, float tanh_alpha, int dtype, zl_stream_t s);
+/* out[r] = tanh(alpha * x[rows[r]]) * w + b of fp32 rows (rows NULL: in order), w, b fp32 (width), out (n_rows, width) in `dtype`. */
+int zls_tanh_norm(const float* x, const int32_t* rows, float alpha, const float* w, const float* b, int64_t n_rows, int64_t width, void* out,
+                  int dtype, zl_stream_t s);
 
 /* ---- a residual kept as several streams ------------------------------------------------------------------------------------------ */
 /* The residual of a token is n <= 8 rows x_0 .. x_{n-1} of `width` fp32 numbers; element (t, s, i) of the streams that are READ lies at

@@ -75,7 +75,7 @@ struct FinP {
     const float* y; const float* m_vals; const float* weight; const float* gate; int64_t ldg;
     int norm_col, heads, vdim, part, g_col0, gate_kind;       // gate_kind 0: sigmoid(gate); 1: silu(gate)
     float q_scale, den_eps, eps;
-    void* out;
+    void* out; int64_t ldo; float out_scale;                  // output rows of ldo numbers, every number times out_scale
 };
 
 template <int DT>
@@ -99,13 +99,13 @@ __global__ __launch_bounds__(kG) void k_linear_attn_finish(const FinP p) {
     const float f = 1.0f / sqrtf(ss / (float)p.part + p.eps);
     for (int i = threadIdx.x; i < p.part; i += blockDim.x) {
         const int c = c0 + i;
-        float v = value(c) * f;
+        float v = value(c) * f * p.out_scale;
         if (p.weight) v *= p.weight[c];
         if (p.gate) {
             const float gv = p.gate[(size_t)t * p.ldg + p.g_col0 + c];
             v *= p.gate_kind == 1 ? seq_silu(gv) : seq_sigmoid(gv);
         }
-        SeqT<DT>::st(p.out, (size_t)t * p.heads * p.vdim + c, v);
+        SeqT<DT>::st(p.out, (size_t)t * p.ldo + c, v);
     }
 }
 
@@ -122,13 +122,13 @@ extern "C" int zls_exp_gates(const float* proj, int64_t ld, int64_t i_col0, int6
 
 extern "C" int zls_linear_attn_finish(const float* y, int64_t norm_col, float q_scale, const float* m_vals, float den_eps, int64_t heads,
                                       int64_t vdim, int64_t norm_groups, const float* weight, float eps, const float* gate, int64_t ldg,
-                                      int64_t g_col0, int64_t n_tok, void* out, int dtype, int gate_kind, zl_stream_t s) {
-    ZL_CHECK_ARG(y && out && heads > 0 && vdim > 0 && norm_groups > 0 && n_tok > 0 && (!m_vals || norm_col), ZL_EINVAL);
+                                      int64_t g_col0, int64_t n_tok, float out_scale, void* out, int64_t ldo, int dtype, int gate_kind, zl_stream_t s) {
+    ZL_CHECK_ARG(y && out && ldo >= heads * vdim && heads > 0 && vdim > 0 && norm_groups > 0 && n_tok > 0 && (!m_vals || norm_col), ZL_EINVAL);
     ZL_CHECK_ARG((heads * vdim) % norm_groups == 0 && norm_groups <= 65535 && (!gate || (g_col0 >= 0 && g_col0 + heads * vdim <= ldg)), ZL_ESHAPE);
     FinP p;
     p.y = y; p.m_vals = m_vals; p.weight = weight; p.gate = gate; p.ldg = ldg; p.norm_col = norm_col ? 1 : 0; p.heads = (int)heads;
     p.vdim = (int)vdim; p.part = (int)(heads * vdim / norm_groups); p.g_col0 = (int)g_col0; p.q_scale = q_scale; p.den_eps = den_eps;
-    p.eps = eps; p.out = out; p.gate_kind = gate_kind == 1 ? 1 : 0;
+    p.eps = eps; p.out = out; p.ldo = ldo; p.out_scale = out_scale; p.gate_kind = gate_kind == 1 ? 1 : 0;
     // (a norm group per workgroup: short groups -- a head each -- get no more waves than they have elements for)
     const unsigned threads = p.part >= kG ? kG : (unsigned)((p.part + 63) / 64 * 64);
 #define CALL(DT) hipLaunchKernelGGL((k_linear_attn_finish<DT>), dim3((unsigned)n_tok, (unsigned)norm_groups), dim3(threads), 0, (hipStream_t)s, p);

@@ -3,7 +3,8 @@
 // norm before a sub-layer (alone, or fused with the residual sum that precedes it), scaled and soft-capped logits, and the same two steps
 // for a residual kept as SEVERAL streams (k_streams_norm, k_streams_update): a sub-layer reads a weighted sum of the streams, its result --
 // optionally gated by a sigmoid -- goes to every stream with a factor of its own while the streams are mixed by a small matrix -- and for
-// sub-layers that run side by side (k_add_branches: normed or plain results join the residual together, two norms of the new row come out).
+// sub-layers that run side by side (k_add_branches: normed or plain results join the residual together, two norms of the new row -- or the
+// tanh norm, which needs no sum over it -- come out).
 // One workgroup per token row; every sum of squares is fp32 (butterfly inside a wave, waves in order).
 #include "seq_common.h"
 
@@ -198,11 +199,13 @@ struct BranchP {
     float eps; int width;
     const float* w1; void* h1; const float* w2; void* h2;
     void* xt; int64_t ldxt;
+    const float* b1; float alpha;                       // the norm without statistics: h1 = tanh(alpha x) * w1 + b1
 };
 
 // x += sum_i coef_i N_i(y_i) of NB branches that ran side by side, and the inputs of the next two sub-layers, both norms of the same new
 // row.  The new row stays in LDS between its sum of squares and its norms; a normed branch is read twice, the second time from L2.
-template <int DT, int NB, int V>
+// TANH: h1 is the norm without statistics (w2 unused), written on the way -- no sum over the row, no LDS, no barrier for it.
+template <int DT, int NB, int V, bool TANH>
 __global__ __launch_bounds__(kT) void k_add_branches(const BranchP p) {
     extern __shared__ __attribute__((aligned(16))) float u[];
     __shared__ float red[16];
@@ -267,12 +270,21 @@ __global__ __launch_bounds__(kT) void k_add_branches(const BranchP p) {
             for (int e = 0; e < V; ++e) x[e] += a[e];
             VecF<V>::st(p.x + row + i, x);
         }
-        VecF<V>::st(u + i, x);
+        if constexpr (TANH) {
+            float a[V], c[V];
+            VecF<V>::ld(p.w1 + i, a);
+            VecF<V>::ld(p.b1 + i, c);
 #pragma unroll
-        for (int e = 0; e < V; ++e) sx = fmaf(x[e], x[e], sx);
+            for (int e = 0; e < V; ++e) a[e] = fmaf(tanhf(p.alpha * x[e]), a[e], c[e]);
+            st_row<DT, V>(p.h1, row + i, a);
+        } else {
+            VecF<V>::st(u + i, x);
+#pragma unroll
+            for (int e = 0; e < V; ++e) sx = fmaf(x[e], x[e], sx);
+        }
         if (p.xt) st_row<DT, V>(p.xt, (size_t)blockIdx.x * p.ldxt + i, x);
     }
-    if (!p.w1 && !p.w2) return;
+    if (TANH || (!p.w1 && !p.w2)) return;
     const float fx = 1.0f / sqrtf(zl_block_sum(sx, red) / (float)p.width + p.eps);
 #pragma unroll 2
     for (int i = threadIdx.x * V; i < p.width; i += kT * V) {                // (a thread reads back its own elements)
@@ -285,6 +297,15 @@ __global__ __launch_bounds__(kT) void k_add_branches(const BranchP p) {
         if (p.w1) st_row<DT, V>(p.h1, row + i, a);
         if (p.w2) st_row<DT, V>(p.h2, row + i, c);
     }
+}
+
+// out[r] = tanh(alpha x[row]) * w + b: a norm that takes no statistics of its row
+template <int DT>
+__global__ __launch_bounds__(kT) void k_tanh_norm(const float* __restrict__ x, const int32_t* __restrict__ rows, float alpha, const float* __restrict__ w,
+                                                  const float* __restrict__ b, int width, void* __restrict__ out) {
+    const size_t src = (size_t)(rows ? rows[blockIdx.x] : (int)blockIdx.x) * width;
+    for (int i = blockIdx.y * kT + threadIdx.x; i < width; i += gridDim.y * kT)
+        SeqT<DT>::st(out, (size_t)blockIdx.x * width + i, fmaf(tanhf(alpha * x[src + i]), w[i], b[i]));
 }
 
 // z <- cap * tanh(z * scale / cap) (cap <= 0: z * scale)
@@ -488,6 +509,17 @@ extern "C" int zls_add_rms_norm(float* x, const float* y, float eps, int64_t row
     return zl_launch_status();
 }
 
+extern "C" int zls_tanh_norm(const float* x, const int32_t* rows, float alpha, const float* w, const float* b, int64_t n_rows, int64_t width, void* out,
+                             int dtype, zl_stream_t s) {
+    ZL_CHECK_ARG(x && w && b && out && n_rows > 0 && width > 0, ZL_EINVAL);
+    const unsigned parts = (unsigned)((width + 4 * kT - 1) / (4 * kT));
+    ZL_CHECK_ARG(parts <= 65535, ZL_ELIMIT);
+#define CALL(DT) hipLaunchKernelGGL((k_tanh_norm<DT>), dim3((unsigned)n_rows, parts), dim3(kT), 0, (hipStream_t)s, x, rows, alpha, w, b, (int)width, out);
+    ZLS_DISPATCH(dtype, CALL)
+#undef CALL
+    return zl_launch_status();
+}
+
 extern "C" int zls_scale_softcap(float* z, int64_t n, float scale, float cap, zl_stream_t s) {
     ZL_CHECK_ARG(z && n > 0 && n < (1LL << 40), ZL_EINVAL);
     hipLaunchKernelGGL(k_scale_softcap, dim3((unsigned)((n + kT - 1) / kT)), dim3(kT), 0, (hipStream_t)s, z, n, scale, cap);
@@ -495,24 +527,27 @@ extern "C" int zls_scale_softcap(float* z, int64_t n, float scale, float cap, zl
 }
 
 extern "C" int zls_add_branches(float* x, const zls_branch_t* branches, int64_t n, float eps, int64_t rows, int64_t width, const float* w1, void* h1,
-                                const float* w2, void* h2, void* xt, int64_t ldxt, int dtype, zl_stream_t s) {
+                                const float* w2, void* h2, void* xt, int64_t ldxt, const float* tanh_b, float tanh_alpha, int dtype, zl_stream_t s) {
+    ZL_CHECK_ARG(!tanh_b || (w1 && !w2), ZL_EINVAL);
     ZL_CHECK_ARG(x && rows > 0 && width > 0 && n >= 0 && (n == 0 || branches) && (!w1 || h1) && (!w2 || h2) && (!xt || ldxt >= width), ZL_EINVAL);
     ZL_CHECK_ARG(n <= kMaxBranches && width * sizeof(float) <= 60 * 1024, ZL_ELIMIT);
     BranchP p = {};
     auto al = [](const void* q) { return ((uintptr_t)q & 15) == 0; };
-    bool vec = width % 4 == 0 && al(x) && al(w1) && al(w2) && al(h1) && al(h2) && al(xt) && (!xt || ldxt % 4 == 0);
+    bool vec = width % 4 == 0 && al(x) && al(w1) && al(w2) && al(h1) && al(h2) && al(tanh_b) && al(xt) && (!xt || ldxt % 4 == 0);
     for (int i = 0; i < n; ++i) {
         ZL_CHECK_ARG(branches[i].y, ZL_EINVAL);
         p.y[i] = branches[i].y; p.w[i] = branches[i].w; p.coef[i] = branches[i].coef;
         vec = vec && al(p.y[i]) && al(p.w[i]);
     }
-    p.x = x; p.eps = eps; p.width = (int)width; p.w1 = w1; p.h1 = h1; p.w2 = w2; p.h2 = h2; p.xt = xt; p.ldxt = ldxt;
+    p.x = x; p.eps = eps; p.width = (int)width; p.w1 = w1; p.h1 = h1; p.w2 = w2; p.h2 = h2; p.xt = xt; p.ldxt = ldxt; p.b1 = tanh_b; p.alpha = tanh_alpha;
     const dim3 grid((unsigned)rows);
     const size_t lds = (size_t)(width + 3) / 4 * 16;
     hipStream_t hs = (hipStream_t)s;
 #define GO(DT, NB)                                                                                 \
-    if (vec) hipLaunchKernelGGL((k_add_branches<DT, NB, 4>), grid, dim3(kT), lds, hs, p);          \
-    else hipLaunchKernelGGL((k_add_branches<DT, NB, 1>), grid, dim3(kT), lds, hs, p);
+    if (tanh_b && vec) hipLaunchKernelGGL((k_add_branches<DT, NB, 4, true>), grid, dim3(kT), 0, hs, p);   \
+    else if (tanh_b) hipLaunchKernelGGL((k_add_branches<DT, NB, 1, true>), grid, dim3(kT), 0, hs, p);     \
+    else if (vec) hipLaunchKernelGGL((k_add_branches<DT, NB, 4, false>), grid, dim3(kT), lds, hs, p);     \
+    else hipLaunchKernelGGL((k_add_branches<DT, NB, 1, false>), grid, dim3(kT), lds, hs, p);
 #define CALL(DT)                                                                                   \
     switch (n) {                                                                                   \
         case 0: GO(DT, 0) break; case 1: GO(DT, 1) break; case 2: GO(DT, 2) break; case 3: GO(DT, 3) break; default: GO(DT, 4) break; \

@@ -35,6 +35,8 @@ struct GemmP {
     // columns once more in the format of x to y2 (nullable): what a following product reads while the rest stays fp32
     const float* bias; int uact;
     void* y2; int64_t ldy2; int n2;
+    // also in EPI instantiations (nullable): after the activation row r is multiplied by row f_rows[r] of a table in the format of x
+    const void* f_table; const int32_t* f_rows; int64_t f_ld; int f_n;
     // few output tiles and a long k: blockIdx.z takes k_part numbers of k and leaves its plain sums in part (parts, m, n); k_split_sum adds them
     float* part; int k_part, n_parts;
 };
@@ -44,6 +46,7 @@ __device__ __forceinline__ void put(const GemmP& p, int row, int col, float v) {
     if constexpr (EPI) {
         if (p.bias) v += p.bias[col];
         if (p.uact >= 0) v = unary_act(v, p.uact);
+        if (p.f_table) v *= SeqT<DT>::ld(p.f_table, (size_t)min(max(p.f_rows[row], 0), p.f_n - 1) * p.f_ld + col);
         if (col < p.n2) SeqT<DT>::st(p.y2, (size_t)row * p.ldy2 + col, v);
     }
     SeqT<ODT>::st(p.y, (size_t)row * p.ldy + col, v);
@@ -410,7 +413,8 @@ int launch(const GemmP& p, hipStream_t hs) {
 extern "C" int zls_version(void) { return 1; }
 
 extern "C" int zls_gemm_nt_act(const void* x, int64_t ldx, const void* w, const float* bias, int act, void* y, int64_t ldy, void* y2, int64_t ldy2,
-                               int64_t n2, int64_t m, int64_t n, int64_t k, float* part, int64_t n_parts, int dtype, int out_dtype, zl_stream_t s) {
+                               int64_t n2, const zls_row_factor_t* factor, int64_t m, int64_t n, int64_t k, float* part, int64_t n_parts, int dtype,
+                               int out_dtype, zl_stream_t s) {
     ZL_CHECK_ARG(x && w && y && m > 0 && n > 0 && k > 0, ZL_EINVAL);
     ZL_CHECK_ARG(ldx >= k && ldy >= n && m < (1 << 30) && n < (1 << 30) && k < (1 << 30), ZL_ESHAPE);
     ZL_CHECK_ARG((m + 63) / 64 <= 65535, ZL_ELIMIT);
@@ -426,11 +430,15 @@ extern "C" int zls_gemm_nt_act(const void* x, int64_t ldx, const void* w, const 
         p.n_parts = (int)((k + p.k_part - 1) / p.k_part);                // (never more than the caller made room for)
         p.part = part;
     }
+    if (factor) {
+        ZL_CHECK_ARG(factor->table && factor->rows && factor->ld >= n && factor->n_rows > 0, ZL_EINVAL);
+        p.f_table = factor->table; p.f_rows = factor->rows; p.f_ld = factor->ld; p.f_n = factor->n_rows;
+    }
     p.bias = bias; p.uact = act; p.y2 = y2; p.ldy2 = ldy2; p.n2 = y2 ? (int)n2 : 0;
     const int64_t unit = dtype == ZL_BF16 ? 8 : 4;
     p.vec = (k % unit == 0 && ldx % unit == 0 && ((uintptr_t)x & 15) == 0 && ((uintptr_t)w & 15) == 0) ? 1 : 0;
     hipStream_t hs = (hipStream_t)s;
-    if (bias || act >= 0 || y2) {
+    if (bias || act >= 0 || y2 || factor) {
         if (dtype == ZL_BF16) return out_dtype == ZL_F32 ? launch<ZL_BF16, ZL_F32, true>(p, hs) : launch<ZL_BF16, ZL_BF16, true>(p, hs);
         return launch<ZL_F32, ZL_F32, true>(p, hs);
     }
@@ -440,7 +448,7 @@ extern "C" int zls_gemm_nt_act(const void* x, int64_t ldx, const void* w, const 
 
 extern "C" int zls_gemm_nt(const void* x, int64_t ldx, const void* w, void* y, int64_t ldy, int64_t m, int64_t n, int64_t k, int dtype,
                            int out_dtype, zl_stream_t s) {
-    return zls_gemm_nt_act(x, ldx, w, nullptr, -1, y, ldy, nullptr, 0, 0, m, n, k, nullptr, 0, dtype, out_dtype, s);
+    return zls_gemm_nt_act(x, ldx, w, nullptr, -1, y, ldy, nullptr, 0, 0, nullptr, m, n, k, nullptr, 0, dtype, out_dtype, s);
 }
 
 // the same product with GATHERED rows of x and / or w (x_rows / w_rows: device int32 row indices, NULL: the rows in order), always on the

@@ -30,13 +30,16 @@ constexpr int kMaxV = 8;            // output coordinates per thread: (all_kv ? 
 // worked out once per token, used by all its heads
 struct Turn {
     float sn[kMaxE], cs[kMaxE];
-    __device__ __forceinline__ void set(int n_rot, const float* __restrict__ freq, float pos, int lane, bool interleaved) {
+    __device__ __forceinline__ void set(int n_rot, const float* __restrict__ freq, float pos, int lane, bool interleaved, float gain = 1.0f) {
         const int half = n_rot >> 1;
 #pragma unroll
         for (int r = 0; r < kMaxE; ++r) {
             const int i = lane + 64 * r;
             sn[r] = 0.f; cs[r] = 1.f;
-            if (i < n_rot) seq_sincos(pos * freq[interleaved ? (i >> 1) : (i < half ? i : i - half)], &sn[r], &cs[r]);
+            if (i < n_rot) {
+                seq_sincos(pos * freq[interleaved ? (i >> 1) : (i < half ? i : i - half)], &sn[r], &cs[r]);
+                sn[r] *= gain; cs[r] *= gain;                            // (rescaled frequencies come with a gain on cos and sin)
+            }
         }
     }
 };
@@ -117,7 +120,7 @@ __global__ __launch_bounds__(256) void k_rope_norm_store(const RopeP p, const zl
         for (int i = threadIdx.x; i < n; i += 256) { const float u = src[i]; ss = fmaf(u, u, ss); }
         f = 1.0f / sqrtf(zl_block_sum(ss, red) / (float)n + p.eps);      // (its barriers: every wave has read the row before one writes it)
     }
-    turn.set(p.rot_dims, p.qk_freq, pos, lane, p.interleaved != 0);
+    turn.set(p.rot_dims, p.qk_freq, pos, lane, p.interleaved != 0, p.prep.rot_gain > 0.f ? p.prep.rot_gain : 1.0f);
     if (queries) {
         const float temp = p.prep.temp_every > 0 ? 1.0f + p.prep.temp_coef * logf((float)((posi + 1) / p.prep.temp_every + 1)) : 1.0f;
         for (int h = wave; h < p.heads; h += 4) {                        // (a wave owns its heads: no two waves touch the same numbers)
@@ -589,6 +592,8 @@ struct MixP {
     void* out;
     const float* sink;                                                    // (heads) nullable: exp(sink_h) joins head h's denominator
     int plain_sum;                                                        // the splits hold finished weights (sigmoids): they are added, not normalised
+    int gate_per_head;                                                    // one gate number per head instead of one per coordinate
+    int64_t ldo; float out_scale;                                         // output rows of ldo numbers, every number times out_scale
 };
 
 // a workgroup per (token, key / value head c): the splits of every source head merged into LDS (for c's values only), then for the heads of
@@ -690,14 +695,17 @@ __global__ __launch_bounds__(256) void k_head_mix_gate(const MixP p, const zls_b
             const float u2 = u * cs + v * sn, v2 = v * cs - u * sn;
             u = u2; v = v2;
         }
-        const size_t o = (size_t)t * p.heads * vd + (size_t)h * vd;
-        if (p.gate) {
+        const size_t o = (size_t)t * p.ldo + (size_t)h * vd;
+        if (p.gate && p.gate_per_head) {
+            const float gv = seq_sigmoid(p.gate[(size_t)t * p.ldg + p.g_col0 + h]);
+            u *= gv; v *= gv;
+        } else if (p.gate) {
             const float* gr = p.gate + (size_t)t * p.ldg + p.g_col0 + h * vd;
             u *= seq_sigmoid(gr[i0]);
             if (i1 < vd) v *= seq_sigmoid(gr[i1]);
         }
-        SeqT<DT>::st(p.out, o + i0, u);
-        if (i1 < vd) SeqT<DT>::st(p.out, o + i1, v);
+        SeqT<DT>::st(p.out, o + i0, u * p.out_scale);
+        if (i1 < vd) SeqT<DT>::st(p.out, o + i1, v * p.out_scale);
     }
 }
 
@@ -813,16 +821,16 @@ extern "C" int zls_window_attention_prompt(const float* q, int64_t ldq, int64_t 
 
 extern "C" int zls_head_mix_gate(const float* acc, const float* ml, int64_t n_splits, const float* talk, const float* v_freq, const float* gate,
                                  int64_t ldg, int64_t g_col0, const float* sink, int plain_sum, const zls_batch_t* b, int64_t heads,
-                                 int64_t kv_heads, int64_t vdim, void* out, int dtype, zl_stream_t s) {
-    ZL_CHECK_ARG(acc && ml && out && seq_batch_ok(b) && heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && vdim > 0 && n_splits >= 1, ZL_EINVAL);
-    ZL_CHECK_ARG((!v_freq || vdim % 2 == 0) && (!gate || (g_col0 >= 0 && g_col0 + heads * vdim <= ldg)), ZL_ESHAPE);
+                                 int64_t kv_heads, int64_t vdim, int gate_per_head, float out_scale, void* out, int64_t ldo, int dtype, zl_stream_t s) {
+    ZL_CHECK_ARG(acc && ml && out && ldo >= heads * vdim && seq_batch_ok(b) && heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && vdim > 0 && n_splits >= 1, ZL_EINVAL);
+    ZL_CHECK_ARG((!v_freq || vdim % 2 == 0) && (!gate || (g_col0 >= 0 && g_col0 + heads * (gate_per_head ? 1 : vdim) <= ldg)), ZL_ESHAPE);
     const int64_t n_src = talk ? heads : heads / kv_heads;
     const size_t lds = (size_t)(n_src * (n_splits + vdim) + (talk ? heads / kv_heads * heads : 0)) * sizeof(float);
     ZL_CHECK_ARG(lds <= 64 * 1024 && kv_heads <= 65535, ZL_ELIMIT);
     MixP p;
     p.acc = acc; p.ml = ml; p.n_splits = (int)n_splits; p.talk = talk; p.v_freq = v_freq; p.gate = gate; p.ldg = ldg; p.g_col0 = (int)g_col0;
     p.heads = (int)heads; p.kv_heads = (int)kv_heads; p.vdim = (int)vdim; p.out = out; p.sink = sink;
-    p.plain_sum = plain_sum ? 1 : 0;
+    p.plain_sum = plain_sum ? 1 : 0; p.gate_per_head = gate_per_head ? 1 : 0; p.ldo = ldo; p.out_scale = out_scale;
 #define CALL(DT) hipLaunchKernelGGL((k_head_mix_gate<DT>), dim3(b->n_tok, (unsigned)kv_heads), dim3(256), lds, (hipStream_t)s, p, *b);
     ZLS_DISPATCH(dtype, CALL)
 #undef CALL

@@ -289,12 +289,13 @@ def linear_slopes(heads, device):
 
 class WindowAttention(SideRows):
     """Softmax attention with grouped key / value heads over a paged cache: rotary positions on the first `rot_dims` coordinates of every
-    query and key head (pairs i, i + rot_dims / 2; every frequency divided by `rot_scaling`), queries and keys divided by their root mean
+    query and key head (pairs i, i + rot_dims / 2; every frequency divided by `rot_scaling`, or rescaled by the dictionary of that name, see
+    scaled_frequencies), queries and keys divided by their root mean
     square afterwards (qk_norm), a sliding window of `window` positions (0: none), optionally
       * values turned by their own position over all vdim coordinates before they are cached and the heads' sums turned back by the query's
         position (rotate_values; frequencies from the same base, never scaled),
       * the heads' softmax weights mixed by a (heads, heads) matrix after the softmax (tensor `talk`),
-      * a sigmoid gate per output coordinate computed from the mixer's input (tensor `g`),
+      * a sigmoid gate per output coordinate computed from the mixer's input (tensor `g`), or per head (head_gate; tensor g (heads, width)),
       * keys and values borrowed from another layer's cache (kv_source: that layer's WindowAttention; then no k / v tensors),
       * rotated pairs that are neighbours (2i, 2i + 1) instead of (i, i + rot_dims / 2) (rope_interleaved),
       * biases on q, k, v (bias; tensors q.b, k.b, v.b) and a short causal convolution over time on every channel of q, k, v right after the
@@ -318,7 +319,7 @@ class WindowAttention(SideRows):
     def __init__(self, name, width, heads, kv_heads, dim, vdim, scale, window, rot_dims, rot_base, rot_scaling, eps, qk_norm=True,
                  rotate_values=True, talk=True, gate=True, kv_source=None, rope_interleaved=False, bias=False, conv_taps=0, keep_first=0,
                  sink=False, v_mix=False, v_mix_source=None, norm_weight=False, head_scale=False, softcap=0.0, rel_far=0, chunk=0,
-                 weights="softmax", whole_norm=False, q_temp=None, slope_bias=False):
+                 weights="softmax", whole_norm=False, q_temp=None, slope_bias=False, head_gate=False):
         if weights not in ("softmax", "sigmoid") or (weights == "sigmoid" and (sink or talk)) or (chunk and keep_first) or chunk < 0:
             raise ZLError("attention: sigmoid weights have no sink and no mixing; chunks keep no first keys")
         if norm_weight and not qk_norm:
@@ -344,8 +345,10 @@ class WindowAttention(SideRows):
         self.sink = self.in_bias = self.conv_w = self.tail = self.last_values = None
         self.vmix_lambda = 0.0
         self.name, self.width, self.heads, self.kv_heads, self.dim, self.vdim = name, width, heads, kv_heads, dim, vdim
-        self.scale, self.window, self.rot_dims, self.rot_base, self.rot_scaling = float(scale), int(window), rot_dims, float(rot_base), float(rot_scaling)
-        self.eps, self.qk_norm, self.rotate_values, self.has_talk, self.has_gate = float(eps), qk_norm, rotate_values, talk, gate
+        self.scale, self.window, self.rot_dims, self.rot_base, self.rot_scaling = float(scale), int(window), rot_dims, float(rot_base), \
+            dict(rot_scaling) if isinstance(rot_scaling, dict) else float(rot_scaling or 1.0)
+        self.eps, self.qk_norm, self.rotate_values, self.has_talk, self.has_gate = float(eps), qk_norm, rotate_values, talk, gate or head_gate
+        self.head_gate, self.rot_gain = bool(head_gate), 1.0
         self.kv_source = kv_source
         self.k_cache = self.v_cache = None
         self.prompt_kernel = True         # bf16 portions on the matrix-core kernel (False: everything on the plain kernel)
@@ -356,10 +359,14 @@ class WindowAttention(SideRows):
         own = self.kv_source is None
         kq, vq = H * d, H * d + (G * d if own else 0)
         g0 = vq + (G * v if own else 0)
-        return kq, vq, g0, g0 + (H * v if self.has_gate else 0)
+        return kq, vq, g0, g0 + (0 if not self.has_gate else H if self.head_gate else H * v)
 
     def _tables(self, device):
-        self.qk_freq = rotary_frequencies(self.rot_dims, self.rot_base, self.rot_scaling, device) if self.rot_dims else None
+        self.qk_freq = None
+        if self.rot_dims and isinstance(self.rot_scaling, dict):
+            self.qk_freq, self.rot_gain = scaled_frequencies(self.rot_dims, self.rot_base, self.rot_scaling, device)
+        elif self.rot_dims:
+            self.qk_freq = rotary_frequencies(self.rot_dims, self.rot_base, self.rot_scaling, device)
         self.v_freq = rotary_frequencies(self.vdim, self.rot_base, 1.0, device) if self.rotate_values else None
         self.form = None
         if self.slope_bias:
@@ -371,8 +378,9 @@ class WindowAttention(SideRows):
     def set_prep(self, extra=None):
         """what the cache-writing launch does besides rotation and norms per head; extra: see seqops.head_prep"""
         self.prep = None
-        if self.whole_norm or self.q_temp or extra:
-            self.prep = seqops.head_prep(self.whole_norm, *((self.q_norm_w, self.k_norm_w) if self.whole_norm else (None, None)), self.q_temp, extra)
+        if self.whole_norm or self.q_temp or extra or self.rot_gain != 1.0:
+            self.prep = seqops.head_prep(self.whole_norm, *((self.q_norm_w, self.k_norm_w) if self.whole_norm else (None, None)), self.q_temp, extra,
+                                         self.rot_gain)
 
     def _load_form(self, get, prefix, device):
         d, H = self.dim, self.heads
@@ -397,7 +405,7 @@ class WindowAttention(SideRows):
         if self.kv_source is None:
             parts += [_mat(get, prefix + "k", (G * d, W), dtype, device), _mat(get, prefix + "v", (G * v, W), dtype, device)]
         if self.has_gate:
-            parts.append(_mat(get, prefix + "g", (H * v, W), dtype, device))
+            parts.append(_mat(get, prefix + "g", (H if self.head_gate else H * v, W), dtype, device))
         self.w_in = torch.cat(parts, dim=0).contiguous()
         self.talk = _mat(get, prefix + "talk", (H, H), torch.float32, device) if self.has_talk else None
         self.w_o = _mat(get, prefix + "o", (W, H * v), dtype, device)
@@ -468,9 +476,15 @@ class WindowAttention(SideRows):
         self.side = (proj, self.side_col0)
         return seqops.gemm_nt(self.attend(proj, 0, batch, h.dtype), self.w_o)
 
-    def attend(self, proj, col0, batch, dtype):
+    def joint_in(self):
+        return None, self.w_in, self.proj_bias
+
+    def joint_out(self):
+        return self.w_o, None
+
+    def attend(self, proj, col0, batch, dtype, lead=None, out=None, out_scale=1.0):
         """everything between the two products, from the fp32 columns [q | k | v | gate] of proj that start at col0 (biases are in them unless
-        a short convolution adds them); returns the output projection's input"""
+        a short convolution adds them); returns the output projection's input, times out_scale, in `out` when given"""
         H, G, d, v = self.heads, self.kv_heads, self.dim, self.vdim
         k0, v0, g0, _ = self._cols()
         own = self.kv_source is None
@@ -489,7 +503,7 @@ class WindowAttention(SideRows):
                                                     all_kv=self.has_talk, mfma=self.prompt_kernel, n_splits=self.n_splits,
                                                     keep_first=self.keep_first, form=self.form)
         return seqops.head_mix_gate(acc, ml, n_splits, self.talk, self.v_freq, proj if self.has_gate else None, col0 + g0, batch, H, G, v, dtype,
-                                    sink=self.sink, plain_sum=self.sigmoid)
+                                    sink=self.sink, plain_sum=self.sigmoid, gate_per_head=self.head_gate, out=out, out_scale=out_scale)
 
 
 class DecayLinearAttention:
@@ -730,6 +744,217 @@ class GatedLinearAttention:
         return seqops.gemm_nt(a, self.w_o)
 
 
+class GatedDeltaRule:
+    """Gated delta rule: q, k, v pass a short causal convolution per channel and SiLU, q and k become unit vectors per head (q times dim^-1/2);
+    beta = sigmoid(W_b h) per head;
+        S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q        per head, S (dim x vdim) fp32 per sequence, from zero
+    with the decay g = exp(-exp(A_log) softplus(z + dt_bias)): decay="head": z = W_a h, a number per head; decay="channel": z = W_a2 (W_a1 h),
+    a number per head and key channel.  Then each head's o is divided by its root mean square over vdim, times a weight shared by the heads,
+    times gate_act of W_g h (gate="full") or of W_g2 (W_g1 h) (gate="lowrank"), and the output projection.  Several heads may share a query /
+    key head.  The two second steps of low-rank pairs are ONE product with a block-diagonal matrix whose input is the LEADING columns of the
+    first product, written once more in the serving format.
+    Tensors under `prefix`: q, k (kv_heads*dim, width), v (heads*vdim, width), q.conv, k.conv, v.conv (channels, taps), b (heads, width), A_log
+    (heads), dt_bias (heads | heads*dim), a (heads, width) or a1 (low, width), a2 (heads*dim, low), g (heads*vdim, width) or g1 (low, width),
+    g2 (heads*vdim, low), norm (vdim), o (width, heads*vdim)."""
+    UNIT_EPS = 1e-6                       # joins a head's sum of squares under the root
+
+    def __init__(self, name, width, heads, kv_heads, dim, vdim, taps, eps, decay="head", gate="full", gate_act="silu"):
+        if heads % kv_heads or min(heads, kv_heads, dim, vdim, taps) < 1:
+            raise ZLError("delta rule: heads must divide by kv_heads, sizes must be positive")
+        if decay not in ("head", "channel") or gate not in ("full", "lowrank") or gate_act not in ("silu", "sigmoid"):
+            raise ZLError("delta rule: decay per head or channel, gate full or lowrank, silu or sigmoid")
+        self.name, self.width, self.heads, self.kv_heads, self.dim, self.vdim, self.taps, self.eps = name, width, heads, kv_heads, dim, vdim, taps, float(eps)
+        self.per_channel, self.lowrank_gate, self.gate_act = decay == "channel", gate == "lowrank", gate_act
+        self.channels = 2 * kv_heads * dim + heads * vdim
+        self.lead = self.w_low = None
+
+    def _pairs(self):
+        """[(first step's name, second step's name, outputs)] of the low-rank pairs"""
+        out = [("a1", "a2", self.heads * self.dim)] if self.per_channel else []
+        return out + ([("g1", "g2", self.heads * self.vdim)] if self.lowrank_gate else [])
+
+    def _rows(self):
+        """[(name, rows)] of the input projection behind the leading low-rank rows"""
+        G, d, H, v = self.kv_heads, self.dim, self.heads, self.vdim
+        return [("q", G * d), ("k", G * d), ("v", H * v), ("b", H)] + ([] if self.per_channel else [("a", H)]) + ([] if self.lowrank_gate else [("g", H * v)])
+
+    def _set(self, mats, firsts, seconds, conv_w, a_log, dt_bias, norm, w_o, device):
+        H, v = self.heads, self.vdim
+        self.w_in = torch.cat(mats, dim=0).contiguous()
+        if firsts:                        # the leading rows, padded to whole 16-byte pieces, and the block-diagonal second step
+            low = sum(m.shape[0] for m in firsts)
+            pad = (low + 7) // 8 * 8
+            self.lead = torch.cat(firsts + [torch.zeros((pad - low, self.width), dtype=firsts[0].dtype, device=device)], dim=0).contiguous()
+            self.w_low = torch.zeros((sum(m.shape[0] for m in seconds), pad), dtype=firsts[0].dtype, device=device)
+            r = c = 0
+            for m in seconds:
+                self.w_low[r:r + m.shape[0], c:c + m.shape[1]] = m
+                r, c = r + m.shape[0], c + m.shape[1]
+        self.conv_w = conv_w.contiguous()
+        self.rate = torch.exp(a_log.double()).to(torch.float32).contiguous()
+        self.dt_bias, self.norm_w, self.w_o = dt_bias, norm.repeat(H).contiguous(), w_o
+        return self
+
+    def load(self, get, prefix, dtype, device):
+        W, H, d, v = self.width, self.heads, self.dim, self.vdim
+        firsts, seconds = [], []
+        for one, two, n in self._pairs():
+            low = int(get(prefix + one).shape[0])
+            firsts.append(_mat(get, prefix + one, (low, W), dtype, device))
+            seconds.append(_mat(get, prefix + two, (n, low), dtype, device))
+        rows = self._rows()
+        conv = torch.cat([_mat(get, prefix + n + ".conv", (r, self.taps), torch.float32, device) for n, r in rows[:3]], dim=0)
+        return self._set([_mat(get, prefix + n, (r, W), dtype, device) for n, r in rows], firsts, seconds, conv, _vec(get, prefix + "A_log", H, device),
+                         _vec(get, prefix + "dt_bias", H * d if self.per_channel else H, device), _vec(get, prefix + "norm", v, device),
+                         _mat(get, prefix + "o", (W, H * v), dtype, device), device)
+
+    def init_random(self, gen, dtype, device, low=None):
+        W, H, d, v = self.width, self.heads, self.dim, self.vdim
+        low = d if low is None else low
+        firsts = [_rand(gen, (low, W), W ** -0.5, dtype, device) for _ in self._pairs()]
+        seconds = [_rand(gen, (n, low), low ** -0.5, dtype, device) for _, _, n in self._pairs()]
+        conv = torch.randn((self.channels, self.taps), generator=gen, device=device) * self.taps ** -0.5
+        return self._set([_rand(gen, (r, W), W ** -0.5, dtype, device) for _, r in self._rows()], firsts, seconds, conv, torch.zeros(H, device=device),
+                         torch.full((H * d if self.per_channel else H,), -3.0, device=device), torch.ones(v, device=device),
+                         _rand(gen, (W, H * v), (H * v) ** -0.5, dtype, device), device)
+
+    def bind(self, cache, dtype):
+        self.tail = cache.add_state(self.name + ".conv", (self.taps - 1, self.channels)) if self.taps > 1 else None
+        self.state = cache.add_state(self.name + ".S", (self.heads, self.vdim, self.dim))     # (a value column's numbers side by side)
+
+    def weight_bytes(self):
+        return sum(t.numel() * t.element_size() for t in (self.w_in, self.lead, self.w_low, self.w_o) if t is not None)
+
+    def joint_in(self):
+        return self.lead, self.w_in, None
+
+    def joint_out(self):
+        return self.w_o, None
+
+    def forward(self, h, batch):
+        if self.lead is None:
+            proj, lead, col0 = seqops.gemm_nt(h, self.w_in), None, 0
+        else:
+            col0 = self.lead.shape[0]
+            proj, lead = seqops.gemm_nt(h, torch.cat([self.lead, self.w_in], dim=0), lead=col0)
+        return seqops.gemm_nt(self.attend(proj, col0, batch, h.dtype, lead=lead), self.w_o)
+
+    def attend(self, proj, col0, batch, dtype, lead=None, out=None, out_scale=1.0):
+        """everything between the two products, from the fp32 columns [q | k | v | b | (a) | (g)] of proj that start at col0 and the low-rank
+        columns `lead` in the serving format; returns the output projection's input, times out_scale, in `out` when given"""
+        H, G, d, v = self.heads, self.kv_heads, self.dim, self.vdim
+        b0 = col0 + self.channels
+        z = seqops.gemm_nt(lead, self.w_low) if self.w_low is not None else None               # fp32 [decay input | gate], the low-rank ones
+        dec, dec0 = (z, 0) if self.per_channel else (proj, b0 + H)
+        gate, gate0 = (z, H * d if self.per_channel else 0) if self.lowrank_gate else (proj, b0 + (H if self.per_channel else 2 * H))
+        qkv, qk, beta, decay = seqops.delta_prep(proj, col0, self.conv_w, self.tail, H, G, d, v, d ** -0.5, self.UNIT_EPS, b0, dec, dec0, self.dt_bias,
+                                                 self.rate, self.per_channel, batch)
+        y = seqops.delta_scan(qkv, qk, beta, decay, self.state, H, G, d, v, batch)
+        return seqops.linear_attn_finish(y, False, 1.0, None, 0.0, H, v, H, self.norm_w, self.eps, gate, gate0, dtype, gate_act=self.gate_act, out=out,
+                                         out_scale=out_scale)
+
+
+class JoinedSublayers:
+    """Sub-layers that read the same input and whose results are added, sum_i scale_i * part_i(h) -- mixers and a feed-forward side by side on
+    one norm -- as TWO products: the parts' input projections are the rows of one matrix, what they leave before their output projections
+    stands side by side in one row, and one matrix of their output projections side by side multiplies and adds it all (the scales act on
+    the fp32 numbers before they are rounded to that row).  A part offers
+        joint_in() -> (lead rows or None, rows, bias or None)      its input projection; lead rows: outputs that are also wanted in the serving format
+        joint_out() -> (matrix, bias or None)                       its output projection
+        attend(proj, col0, batch, dtype, lead, out, out_scale)      everything between, from its columns of proj into its columns of the row
+    parts: [(tensor prefix, part, scale)]; name + part names register the caches and states."""
+
+    def __init__(self, width, parts):
+        self.width, self.parts = width, [p for _, p, _ in parts]
+        self.prefixes, self.scales = [n for n, _, _ in parts], [float(s) for _, _, s in parts]
+        if any(p.width != width for p in self.parts):
+            raise ZLError("joined sub-layers: one width")
+
+    def load(self, get, prefix, dtype, device):
+        for n, p in zip(self.prefixes, self.parts):
+            p.load(get, prefix + n, dtype, device)
+        return self._join()
+
+    def init_random(self, gen, dtype, device):
+        for p in self.parts:
+            p.init_random(gen, dtype, device)
+        return self._join()
+
+    def _join(self):
+        leads, rows, biases = zip(*[p.joint_in() for p in self.parts])
+        self.n_lead = sum(m.shape[0] for m in leads if m is not None)
+        self.w_in = torch.cat([m for m in leads if m is not None] + list(rows), dim=0).contiguous()
+        self.in_bias = None
+        if any(b is not None for b in biases):
+            self.in_bias = torch.zeros(self.w_in.shape[0], device=self.w_in.device)
+        self.lead_at, self.col0, lead_at, at = [], [], 0, self.n_lead
+        for lead, r, b in zip(leads, rows, biases):
+            self.lead_at.append(None if lead is None else (lead_at, lead_at + lead.shape[0]))
+            self.col0.append(at)
+            if b is not None:
+                self.in_bias[at:at + b.numel()] = b
+            lead_at, at = lead_at + (0 if lead is None else lead.shape[0]), at + r.shape[0]
+        mats, biases = zip(*[p.joint_out() for p in self.parts])
+        self.w_out = torch.cat(mats, dim=1).contiguous()
+        self.out_at, at = [], 0
+        for m in mats:
+            self.out_at.append((at, at + m.shape[1]))
+            at += m.shape[1]
+        self.out_bias = None
+        for b, s in zip(biases, self.scales):
+            if b is not None:
+                self.out_bias = b * s if self.out_bias is None else self.out_bias + b * s
+        for p in self.parts:                                                      # (the rows live in the joint matrices now)
+            for n in ("w_in", "lead", "w_gu", "w_o", "w_down"):
+                if getattr(p, n, None) is not None:
+                    setattr(p, n, None)
+        return self
+
+    def bind(self, cache, dtype):
+        for p in self.parts:
+            p.bind(cache, dtype)
+
+    def weight_bytes(self):
+        extra = [getattr(p, "w_low", None) for p in self.parts]
+        return sum(t.numel() * t.element_size() for t in [self.w_in, self.w_out] + extra if t is not None)
+
+    def forward(self, h, batch):
+        proj, lead = seqops.gemm_nt(h, self.w_in, bias=self.in_bias, lead=self.n_lead) if self.n_lead else (seqops.gemm_nt(h, self.w_in, bias=self.in_bias), None)
+        row = torch.empty((batch.n_tok, self.w_out.shape[1]), dtype=h.dtype, device=h.device)
+        for p, s, c, l, (a, b) in zip(self.parts, self.scales, self.col0, self.lead_at, self.out_at):
+            p.attend(proj, c, batch, h.dtype, lead=None if l is None else lead[:, l[0]:l[1]], out=row[:, a:b], out_scale=s)
+        return seqops.gemm_nt(row, self.w_out, bias=self.out_bias)
+
+
+class TokenSideInput:
+    """A second embedding that enters the residual behind a layer: e = dim columns of a table, looked up by the token; y = W_proj (gelu_tanh(W_gate x)
+    * e), in the tanh form, joins the residual with an RMS norm over the model width.  The activation and the product with e are in the
+    first product's epilogue.  Tensors under `prefix`: gate (dim, width), proj (width, dim), norm (width)."""
+
+    def __init__(self, width, dim, column):
+        self.width, self.dim, self.column = width, dim, column
+
+    def load(self, get, prefix, dtype, device):
+        self.w_gate = _mat(get, prefix + "gate", (self.dim, self.width), dtype, device)
+        self.w_proj = _mat(get, prefix + "proj", (self.width, self.dim), dtype, device)
+        self.norm_w = _vec(get, prefix + "norm", self.width, device)
+        return self
+
+    def init_random(self, gen, dtype, device):
+        self.w_gate = _rand(gen, (self.dim, self.width), self.width ** -0.5, dtype, device)
+        self.w_proj = _rand(gen, (self.width, self.dim), self.dim ** -0.5, dtype, device)
+        self.norm_w = 1.0 + 0.1 * torch.randn(self.width, generator=gen, device=device)
+        return self
+
+    def weight_bytes(self):
+        return sum(t.numel() * t.element_size() for t in (self.w_gate, self.w_proj))
+
+    def branch(self, xt, table, tokens, coef):
+        """xt: the residual in the serving format; table (vocab, columns); the branch that seqops.add_branches sums"""
+        g = seqops.gemm_nt(xt, self.w_gate, out_dtype=xt.dtype, act="gelu_tanh", factor=(table, self.column, tokens))
+        return seqops.gemm_nt(g, self.w_proj), self.norm_w, coef
+
+
 class PlainFF(SideRows):
     """Dense feed-forward down(act(up h)) without biases and without a gate; act: "relu2" (the square of relu), "gelu_tanh" or "silu".
     Tensors under `prefix`: up (ff, width), down (width, ff)."""
@@ -762,30 +987,51 @@ class PlainFF(SideRows):
 
 
 class GatedFF:
-    """Dense gated feed-forward down(act(gate h) * (up h)) without biases; act: "gelu_tanh" (the tanh form) or "silu".
-    Tensors under `prefix`: gate, up (ff, width), down (width, ff).  gate | up are one product."""
+    """Dense gated feed-forward down(act(gate h) * (up h)); act: "gelu_tanh" (the tanh form) or "silu"; bias: every projection has one (tensors
+    gate.b, up.b (ff), down.b (width)).  Tensors under `prefix`: gate, up (ff, width), down (width, ff).  gate | up are one product."""
+    in_bias = out_bias = None
 
-    def __init__(self, width, ff, act="gelu_tanh"):
+    def __init__(self, width, ff, act="gelu_tanh", bias=False):
         if act not in ("gelu_tanh", "silu"):
             raise ZLError(f"feed-forward: unknown activation {act!r}")
-        self.width, self.ff, self.act = width, ff, act
+        self.width, self.ff, self.act, self.has_bias = width, ff, act, bool(bias)
 
     def load(self, get, prefix, dtype, device):
         self.w_gu = torch.cat([_mat(get, prefix + "gate", (self.ff, self.width), dtype, device),
                                _mat(get, prefix + "up", (self.ff, self.width), dtype, device)], dim=0).contiguous()
         self.w_down = _mat(get, prefix + "down", (self.width, self.ff), dtype, device)
+        if self.has_bias:
+            self.in_bias = torch.cat([_vec(get, prefix + n + ".b", self.ff, device) for n in ("gate", "up")]).contiguous()
+            self.out_bias = _vec(get, prefix + "down.b", self.width, device)
         return self
 
     def init_random(self, gen, dtype, device):
         self.w_gu = _rand(gen, (2 * self.ff, self.width), self.width ** -0.5, dtype, device)
         self.w_down = _rand(gen, (self.width, self.ff), self.ff ** -0.5, dtype, device)
+        if self.has_bias:
+            self.in_bias, self.out_bias = (0.1 * torch.randn(n, generator=gen, device=device) for n in (2 * self.ff, self.width))
         return self
 
     def weight_bytes(self):
         return sum(t.numel() * t.element_size() for t in (self.w_gu, self.w_down))
 
     def forward(self, h):
-        return seqops.gemm_nt(seqops.act_mul(seqops.gemm_nt(h, self.w_gu), h.dtype, kind=self.act), self.w_down)
+        return seqops.gemm_nt(seqops.act_mul(seqops.gemm_nt(h, self.w_gu, bias=self.in_bias), h.dtype, kind=self.act), self.w_down, bias=self.out_bias)
+
+    def bind(self, cache, dtype):
+        pass
+
+    def joint_in(self):
+        return None, self.w_gu, self.in_bias
+
+    def joint_out(self):
+        return self.w_down, self.out_bias
+
+    def attend(self, proj, col0, batch, dtype, lead=None, out=None, out_scale=1.0):
+        """what lies between the two products, from the columns [gate | up] of proj that start at col0"""
+        if out_scale != 1.0:
+            raise ZLError("feed-forward: no output scale")
+        return seqops.act_mul(proj, dtype, kind=self.act, col0=col0, ff=self.ff, out=out)
 
 
 class MLSTMMixer:

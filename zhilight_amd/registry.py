@@ -27,6 +27,7 @@ def _ensure_builtin():
     from . import gutivik  # noqa: F401
     from . import gaparax  # noqa: F401
     from . import zasazen  # noqa: F401
+    from . import suvapel  # noqa: F401
     from . import llama    # noqa: F401
 
 

@@ -21,7 +21,7 @@ SYMBOLS = ["zls_version", "zls_gemm_nt", "zls_gemm_nt_act", "zls_embed", "zls_to
            "zls_add_layer_norm", "zls_rope_norm_store", "zls_window_attention", "zls_window_attention_prompt", "zls_head_mix_gate", "zls_decay_scan", "zls_exp_gates",
            "zls_linear_attn_finish", "zls_moe_route", "zls_moe_align", "zls_gemm_nt_grouped", "zls_silu_mul", "zls_moe_combine", "zls_rms_norm",
            "zls_add_rms_norm", "zls_scale_softcap", "zls_act_mul", "zls_short_conv", "zls_lowrank_decay", "zls_latent_rope_store",
-           "zls_streams_norm", "zls_streams_update", "zls_unary_act", "zls_add_branches"]
+           "zls_streams_norm", "zls_streams_update", "zls_unary_act", "zls_add_branches", "zls_tanh_norm", "zls_delta_prep", "zls_delta_scan"]
 _STATUS = {-1: "invalid argument (null pointer / non-positive size)", -2: "shape not supported", -3: "dtype not supported",
            -4: "exceeds a hardware limit"}
 
@@ -42,7 +42,12 @@ class ScoreForm(C.Structure):
 class HeadPrep(C.Structure):
     """zls_head_prep_t"""
     _fields_ = [("whole_norm", C.c_int32), ("q_w", C.c_void_p), ("k_w", C.c_void_p), ("temp_coef", C.c_float), ("temp_every", C.c_int32),
-                ("x_col0", C.c_int32), ("x_heads", C.c_int32), ("x_dim", C.c_int32), ("x_rot", C.c_int32), ("x_freq", C.c_void_p)]
+                ("x_col0", C.c_int32), ("x_heads", C.c_int32), ("x_dim", C.c_int32), ("x_rot", C.c_int32), ("x_freq", C.c_void_p), ("rot_gain", C.c_float)]
+
+
+class RowFactor(C.Structure):
+    """zls_row_factor_t"""
+    _fields_ = [("table", C.c_void_p), ("rows", C.c_void_p), ("ld", C.c_int64), ("n_rows", C.c_int32)]
 
 
 _lib = None
@@ -193,9 +198,10 @@ def _k_parts(m, n, k):
     return 1 if tiles > 256 else max(1, min(512 // tiles, k // 256, 16))
 
 
-def gemm_nt(x, w, out=None, out_dtype=torch.float32, bias=None, act=None, lead=0):
+def gemm_nt(x, w, out=None, out_dtype=torch.float32, bias=None, act=None, lead=0, factor=None):
     """act(x (m, k) . w (n, k)^T + bias) -> (m, n); x and w in the serving format, the result fp32 (or that format); bias fp32 (n) or None,
-    act one of UNARY_ACTS or None.  lead > 0: returns (result, its leading `lead` columns once more in the serving format)"""
+    act one of UNARY_ACTS or None.  lead > 0: returns (result, its leading `lead` columns once more in the serving format).  factor =
+    (table, column, rows): result row r is multiplied, after act, by the n numbers of table[rows[r]] from that column"""
     _cuda(w, bias)
     _f32(bias)
     if x.dim() != 2 or x.stride(1) != 1 or not x.is_cuda:
@@ -211,10 +217,17 @@ def gemm_nt(x, w, out=None, out_dtype=torch.float32, bias=None, act=None, lead=0
     elif out.shape != (m, n) or not out.is_contiguous():
         raise ZLError("gemm_nt: wrong output")
     y2 = torch.empty((m, lead), dtype=x.dtype, device=x.device) if lead > 0 else None
+    f = None
+    if factor is not None:
+        table, col, rows = factor
+        _cuda(table, rows)
+        if table.dim() != 2 or table.dtype != x.dtype or col < 0 or col + n > table.shape[1] or rows.dtype != torch.int32 or rows.numel() != m:
+            raise ZLError("gemm_nt: the factor is n columns of a table in the serving format, one row index (int32) per result row")
+        f = C.byref(RowFactor(table.data_ptr() + col * table.element_size(), rows.data_ptr(), table.shape[1], table.shape[0]))
     parts = _k_parts(m, n, k)
     part = torch.empty((parts, m, n), dtype=torch.float32, device=x.device) if parts > 1 else None
     check(lib().zls_gemm_nt_act(_p(x), _i(x.stride(0)), _p(w), _p(bias), C.c_int(-1 if act is None else UNARY_ACTS[act]), _p(out), _i(n), _p(y2),
-                                _i(lead), _i(lead), _i(m), _i(n), _i(k), _p(part), _i(parts), C.c_int(dt_code(x.dtype)), C.c_int(dt_code(out.dtype)), _stream()), "gemm_nt")
+                                _i(lead), _i(lead), f, _i(m), _i(n), _i(k), _p(part), _i(parts), C.c_int(dt_code(x.dtype)), C.c_int(dt_code(out.dtype)), _stream()), "gemm_nt")
     return (out, y2) if lead > 0 else out
 
 
@@ -491,23 +504,41 @@ class Branch(C.Structure):
     _fields_ = [("y", C.c_void_p), ("w", C.c_void_p), ("coef", C.c_float)]
 
 
-def add_branches(x, branches, eps, dtype, weight1=None, weight2=None, xt=None):
+def add_branches(x, branches, eps, dtype, weight1=None, weight2=None, xt=None, tanh=None):
     """x += sum of coef * N(y) over branches = [(y, w or None, coef)] in place (w None: y as it is; no branches: x stays); returns (h1, h2) =
     the RMS norms of the new x with weight1 / weight2 in `dtype` (None without the weight); xt: a (rows, width) view of unit column stride
-    that receives the new x in its own format"""
-    _cuda(x, weight1, weight2, *[t for b in branches for t in b[:2]])
-    _f32(x, weight1, weight2, *[t for b in branches for t in b[:2]])
+    that receives the new x in its own format; tanh = (alpha, b): h1 = tanh(alpha x) * weight1 + b instead (no weight2)"""
+    alpha, shift = tanh if tanh is not None else (0.0, None)
+    _cuda(x, weight1, weight2, shift, *[t for b in branches for t in b[:2]])
+    _f32(x, weight1, weight2, shift, *[t for b in branches for t in b[:2]])
     rows, width = x.shape
     for y, w, _ in branches:
         if y.shape != x.shape or (w is not None and w.numel() != width):
             raise ZLError("add_branches: shape mismatch")
+    if any(t is not None and t.numel() != width for t in (weight1, weight2, shift)):
+        raise ZLError("add_branches: one weight per column")
     if xt is not None and (xt.shape != x.shape or xt.stride(1) != 1 or xt.dtype != dtype or not xt.is_cuda):
         raise ZLError("add_branches: xt must be rows of x's shape in the serving format")
     h1, h2 = (torch.empty((rows, width), dtype=dtype, device=x.device) if w is not None else None for w in (weight1, weight2))
     arr = (Branch * max(1, len(branches)))(*[Branch(y.data_ptr(), 0 if w is None else w.data_ptr(), float(c)) for y, w, c in branches])
     check(lib().zls_add_branches(_p(x), arr, _i(len(branches)), _f(eps), _i(rows), _i(width), _p(weight1), _p(h1), _p(weight2), _p(h2), _p(xt),
-                                 _i(0 if xt is None else xt.stride(0)), C.c_int(dt_code(dtype)), _stream()), "add_branches")
+                                 _i(0 if xt is None else xt.stride(0)), _p(shift), _f(alpha), C.c_int(dt_code(dtype)), _stream()), "add_branches")
     return h1, h2
+
+
+def tanh_norm(x, weight, bias, alpha, dtype, rows=None):
+    """tanh(alpha x) * weight + bias of the rows `rows` (int32 device; None: all) of fp32 x, in `dtype`"""
+    _cuda(x, weight, bias, rows)
+    _f32(x, weight, bias)
+    if rows is not None and rows.dtype != torch.int32:
+        raise ZLError("tanh_norm: rows must be int32")
+    if weight.numel() != x.shape[1] or bias.numel() != x.shape[1]:
+        raise ZLError("tanh_norm: one weight and one bias per column")
+    n = x.shape[0] if rows is None else rows.numel()
+    out = torch.empty((n, x.shape[1]), dtype=dtype, device=x.device)
+    check(lib().zls_tanh_norm(_p(x), _p(rows), _f(alpha), _p(weight), _p(bias), _i(n), _i(x.shape[1]), _p(out), C.c_int(dt_code(dtype)), _stream()),
+          "tanh_norm")
+    return out
 
 
 # ---- a residual kept as several streams ------------------------------------------------------------------------------------------------
@@ -572,10 +603,11 @@ def scale_softcap(z, scale, cap):
 
 
 # ---- softmax attention over paged keys and values -------------------------------------------------------------------------------------------
-def head_prep(whole_norm=False, q_w=None, k_w=None, temp=None, extra=None):
+def head_prep(whole_norm=False, q_w=None, k_w=None, temp=None, extra=None, rot_gain=1.0):
     """The optional parts of rope_norm_store: one norm over all query (key) heads of a token with a weight per number (q_w, k_w fp32), before
     the rotation; temp = (coef, every): queries times 1 + coef ln(floor((p + 1) / every) + 1); extra = (column, heads, dim, rotated
-    coordinates, frequencies): further heads of the same rows that are rotated in place.  Keeps the tensors alive."""
+    coordinates, frequencies): further heads of the same rows that are rotated in place; rot_gain: a factor on the queries' and keys' cos and sin.
+    Keeps the tensors alive."""
     _cuda(q_w, k_w)
     _f32(q_w, k_w)
     coef, every = temp if temp else (0.0, 0)
@@ -585,7 +617,7 @@ def head_prep(whole_norm=False, q_w=None, k_w=None, temp=None, extra=None):
     if freq is not None and freq.numel() != rot // 2 or (rot and freq is None):
         raise ZLError("head_prep: one frequency per rotated pair")
     h = HeadPrep(int(bool(whole_norm)), 0 if q_w is None else q_w.data_ptr(), 0 if k_w is None else k_w.data_ptr(), float(coef), int(every),
-                 int(col), int(heads), int(dim), int(rot), 0 if freq is None else freq.data_ptr())
+                 int(col), int(heads), int(dim), int(rot), 0 if freq is None else freq.data_ptr(), float(rot_gain))
     h.keep, h.sizes = (q_w, k_w, freq), (0 if q_w is None else q_w.numel(), 0 if k_w is None else k_w.numel())
     return h
 
@@ -675,7 +707,19 @@ def window_attention(q, q_col0, k_cache, v_cache, batch, scale, window, heads, k
     return acc, ml, n_splits
 
 
-def head_mix_gate(acc, ml, n_splits, talk, v_freq, gate, g_col0, batch, heads, kv_heads, vdim, dtype, sink=None, plain_sum=False):
+def _out_rows(out, n_tok, width, dtype, device):
+    """a fresh (n_tok, width) result, or the caller's rows of unit column stride (columns of a wider buffer)"""
+    if out is None:
+        return torch.empty((n_tok, width), dtype=dtype, device=device)
+    if tuple(out.shape) != (n_tok, width) or out.stride(1) != 1 or out.dtype != dtype or not out.is_cuda:
+        raise ZLError("the given output must be rows of the result's shape and format")
+    return out
+
+
+def head_mix_gate(acc, ml, n_splits, talk, v_freq, gate, g_col0, batch, heads, kv_heads, vdim, dtype, sink=None, plain_sum=False, gate_per_head=False,
+                  out=None, out_scale=1.0):
+    """the merged heads' sums, mixed (talk), turned back (v_freq), times the sigmoid gate -- a number per coordinate or per head
+    (gate_per_head) --, times out_scale, in `dtype`; out: rows to write into (None: fresh ones)"""
     _cuda(acc, ml, talk, v_freq, gate, sink)
     _f32(acc, ml, talk, v_freq, gate, sink)
     if sink is not None and sink.numel() != heads:
@@ -684,10 +728,10 @@ def head_mix_gate(acc, ml, n_splits, talk, v_freq, gate, g_col0, batch, heads, k
         raise ZLError("head_mix_gate: the mixing matrix is (heads, heads)")
     if acc.numel() != batch.n_tok * heads * n_splits * (kv_heads if talk is not None else 1) * vdim or ml.numel() != batch.n_tok * heads * n_splits * 2:
         raise ZLError("head_mix_gate: acc / ml do not fit")
-    out = torch.empty((batch.n_tok, heads * vdim), dtype=dtype, device=acc.device)
+    out = _out_rows(out, batch.n_tok, heads * vdim, dtype, acc.device)
     check(lib().zls_head_mix_gate(_p(acc), _p(ml), _i(n_splits), _p(talk), _p(v_freq), _p(gate), _i(0 if gate is None else gate.shape[1]),
-                                  _i(g_col0), _p(sink), C.c_int(int(plain_sum)), batch.ref, _i(heads), _i(kv_heads), _i(vdim), _p(out), C.c_int(dt_code(dtype)),
-                                  _stream()), "head_mix_gate")
+                                  _i(g_col0), _p(sink), C.c_int(int(plain_sum)), batch.ref, _i(heads), _i(kv_heads), _i(vdim),
+                                  C.c_int(int(gate_per_head)), _f(out_scale), _p(out), _i(out.stride(0)), C.c_int(dt_code(dtype)), _stream()), "head_mix_gate")
     return out
 
 
@@ -739,17 +783,54 @@ def lowrank_decay(proj, u_col0, w2, bias, tau):
     return alpha
 
 
-def linear_attn_finish(y, norm_col, q_scale, m_vals, den_eps, heads, vdim, norm_groups, weight, eps, gate, g_col0, dtype, gate_act="sigmoid"):
+def linear_attn_finish(y, norm_col, q_scale, m_vals, den_eps, heads, vdim, norm_groups, weight, eps, gate, g_col0, dtype, gate_act="sigmoid", out=None,
+                       out_scale=1.0):
     _cuda(y, m_vals, weight, gate)
     _f32(y, m_vals, weight, gate)
     n_tok = y.shape[0]
     if y.shape[1] != heads * (vdim + (1 if norm_col else 0)):
         raise ZLError("linear_attn_finish: y does not fit")
-    out = torch.empty((n_tok, heads * vdim), dtype=dtype, device=y.device)
+    out = _out_rows(out, n_tok, heads * vdim, dtype, y.device)
     check(lib().zls_linear_attn_finish(_p(y), _i(int(norm_col)), _f(q_scale), _p(m_vals), _f(den_eps), _i(heads), _i(vdim), _i(norm_groups),
-                                       _p(weight), _f(eps), _p(gate), _i(0 if gate is None else gate.shape[1]), _i(g_col0), _i(n_tok), _p(out),
+                                       _p(weight), _f(eps), _p(gate), _i(0 if gate is None else gate.shape[1]), _i(g_col0), _i(n_tok), _f(out_scale), _p(out), _i(out.stride(0)),
                                        C.c_int(dt_code(dtype)), C.c_int(1 if gate_act == "silu" else 0), _stream()), "linear_attn_finish")
     return out
+
+
+# ---- gated delta rule --------------------------------------------------------------------------------------------------------------------
+def delta_prep(proj, col0, conv_w, tail, heads, kv_heads, dim, vdim, q_scale, unit_eps, b_col0, z, z_col0, z_bias, rate, per_channel, batch):
+    """convolution + SiLU, unit vectors, q . k, beta and decays of a step: (qkv, qk, beta, decay) for delta_scan; the carried tail moves on"""
+    _cuda(proj, conv_w, tail, z, z_bias, rate)
+    _f32(proj, conv_w, tail, z, z_bias, rate)
+    channels, taps = conv_w.shape
+    D = heads * dim if per_channel else heads
+    if channels != 2 * kv_heads * dim + heads * vdim or (tail is not None and tuple(tail.shape[1:]) != (taps - 1, channels)):
+        raise ZLError("delta_prep: the convolution covers q, k and v; its tail is (slots, taps - 1, channels)")
+    if rate.numel() != heads or (z_bias is not None and z_bias.numel() != D) or z.shape[0] != proj.shape[0] or proj.shape[0] != batch.n_tok:
+        raise ZLError("delta_prep: shapes")
+    n, dev = batch.n_tok, proj.device
+    qkv, qk = torch.empty((n, channels), dtype=torch.float32, device=dev), torch.empty((n, kv_heads), dtype=torch.float32, device=dev)
+    beta, decay = torch.empty((n, heads), dtype=torch.float32, device=dev), torch.empty((n, D), dtype=torch.float32, device=dev)
+    check(lib().zls_delta_prep(_p(proj), _i(proj.shape[1]), _i(col0), _p(conv_w), _p(tail), _i(taps), _i(heads), _i(kv_heads), _i(dim), _i(vdim),
+                               _f(q_scale), _f(unit_eps), _i(b_col0), _p(z), _i(z.shape[1]), _i(z_col0), _p(z_bias), _p(rate),
+                               C.c_int(int(per_channel)), batch.ref, _p(qkv), _p(qk), _p(beta), _p(decay), _stream()), "delta_prep")
+    return qkv, qk, beta, decay
+
+
+def delta_scan(qkv, qk, beta, decay, state, heads, kv_heads, dim, vdim, batch):
+    """S <- g S; u = beta (v - S^T k); S <- S + k u^T; y = S^T q over the step's portions: fp32 y (n_tok, heads * vdim); state (slots, heads,
+    vdim, dim) moves on.  decay (n_tok, heads) or, per key channel, (n_tok, heads * dim)"""
+    _cuda(qkv, qk, beta, decay, state)
+    _f32(qkv, qk, beta, decay, state)
+    n = batch.n_tok
+    per_channel = decay.shape[1] == heads * dim and dim > 1
+    if tuple(qkv.shape) != (n, 2 * kv_heads * dim + heads * vdim) or tuple(qk.shape) != (n, kv_heads) or tuple(beta.shape) != (n, heads) or \
+            tuple(decay.shape) != (n, heads * dim if per_channel else heads) or tuple(state.shape[1:]) != (heads, vdim, dim):
+        raise ZLError("delta_scan: shapes")
+    y = torch.empty((n, heads * vdim), dtype=torch.float32, device=qkv.device)
+    check(lib().zls_delta_scan(_p(qkv), _p(qk), _p(beta), _p(decay), C.c_int(int(per_channel)), _p(state), _i(heads), _i(kv_heads), _i(dim),
+                               _i(vdim), batch.ref, _p(y), _stream()), "delta_scan")
+    return y
 
 
 # ---- mixture of experts ------------------------------------------------------------------------------------------------------------------
@@ -825,18 +906,18 @@ def silu_mul(gu, dtype):
     return out
 
 
-def act_mul(gu, dtype, kind="silu", alpha=1.0, limit=0.0, block=0, col0=0, ff=None):
+def act_mul(gu, dtype, kind="silu", alpha=1.0, limit=0.0, block=0, col0=0, ff=None, out=None):
     """act(gate, up) of fp32 rows [gates | ups] (block 0) or blocks of `block` gates followed by their ups; see ACT_KINDS.  ff: the 2 ff
-    columns from col0 of wider rows (None: all columns)"""
+    columns from col0 of wider rows (None: all columns); out: rows to write into (None: fresh ones)"""
     _cuda(gu)
     _f32(gu)
     rows, ld = gu.shape
     ff = ld // 2 if ff is None else ff
     if col0 < 0 or col0 + 2 * ff > ld:
         raise ZLError("act_mul: columns")
-    out = torch.empty((rows, ff), dtype=dtype, device=gu.device)
+    out = _out_rows(out, rows, ff, dtype, gu.device)
     check(lib().zls_act_mul(C.c_void_p(gu.data_ptr() + 4 * col0), _i(ld), _i(rows), _i(ff), C.c_int(ACT_KINDS[kind]), _f(alpha), _f(limit), _i(block),
-                            _p(out), C.c_int(dt_code(dtype)), _stream()), "act_mul")
+                            _p(out), _i(out.stride(0)), C.c_int(dt_code(dtype)), _stream()), "act_mul")
     return out
 
 
