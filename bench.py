@@ -21,6 +21,7 @@ fields, `roofline` (the W4A16 GEMV kernel: algorithmic bytes / HIP-event time, v
     python bench.py --gutivik 1b,8b [--seq 2048]
     python bench.py --gaparax 1b,8b [--seq 2048] [--only TEXT]
     python bench.py --zasazen 1b,8b [--seq 2048] [--only TEXT]
+    python bench.py --suvapel 1b,8b [--seq 2048] [--only TEXT]
 
 is a different measurement with its own JSON line: prefill / decode throughput of the ragged-step engine's latent-attention, state-space
 and hybrid stacks (zhilight_amd/tupitar.py) beside the dense bf16 Llama-shaped stack of equal width, 4 layers each, random weights;
@@ -28,6 +29,7 @@ and hybrid stacks (zhilight_amd/tupitar.py) beside the dense bf16 Llama-shaped s
 --gutivik the same for the Gutivik stacks (zhilight_amd/gutivik.py) beside Retotar stacks of equal width.
 --gaparax the same for the Gaparax stacks (zhilight_amd/gaparax.py) beside Gutivik stacks of equal width.
 --zasazen the same for the Zasazen stacks (zhilight_amd/zasazen.py) beside Gutivik, Retotar and Tupitar stacks of equal width.
+--suvapel the same for the Suvapel stacks (zhilight_amd/suvapel.py) beside Gutivik and Zasazen stacks of equal width.
 """
 import argparse
 import json
@@ -846,6 +848,54 @@ def bench_zasazen(args, dev):
     print(json.dumps({"metric": "zasazen_throughput", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "layers": 4, "results": results}))
 
 
+SUVAPEL_BENCH_SIZES = {
+    # name: width; attention heads / key-value heads x head size, window, kept first keys, taps; delta-rule heads / query-key heads x key size x
+    #       value size; the dense feed-forward's ff; columns of the per-layer token input.  Head counts and sizes are those of the sizes of the
+    #       same name above.
+    "1b": dict(width=2048, heads=16, kv_heads=4, dim=128, window=1024, keep=4, rot=64, taps=4, d_heads=16, d_kv=8, d_dim=128, d_vdim=128, ff=5440, side=256),
+    "8b": dict(width=4096, heads=32, kv_heads=8, dim=128, window=1024, keep=4, rot=64, taps=4, d_heads=32, d_kv=16, d_dim=128, d_vdim=128, ff=9536, side=256),
+}
+
+
+def bench_suvapel(args, dev):
+    """--suvapel: prefill and decode throughput of Suvapel stacks (zhilight_amd/suvapel.py: mixers and feed-forward side by side on one norm;
+    a gated delta rule alone, or with a decay per key channel beside windowed attention with kept first keys; a per-layer token input) beside
+    the closest existing models of equal width -- Gutivik's windowed attention and gated linear attention (a decay per key channel) with
+    dense feed-forwards of the same size, Zasazen's attention beside a retention layer --, 4 layers each, random weights, bf16, eager
+    launches.  One JSON line."""
+    from zhilight_amd.gutivik import GutivikConfig, GutivikLayerConfig, GutivikModel
+    from zhilight_amd.suvapel import SuvapelConfig, SuvapelLayerConfig, SuvapelModel
+    from zhilight_amd.zasazen import ZasazenConfig, ZasazenLayerConfig, ZasazenModel
+    seq, vocab, results = args.seq, 32000, []
+
+    def measure(label, name, build):
+        if args.only and args.only not in label:
+            return
+        model = build().init_random(1)
+        _measure_ragged(results, label, name, model, seq, vocab)
+
+    for name in args.suvapel.split(","):
+        z = SUVAPEL_BENCH_SIZES[name]
+        W, dense = z["width"], dict(kind="dense", ff=z["ff"])
+        att = dict(heads=z["heads"], kv_heads=z["kv_heads"], dim=z["dim"], vdim=z["dim"], scale=z["dim"] ** -0.5, conv=z["taps"],
+                   mask=dict(size=z["window"], keep_first=z["keep"]), rot=dict(dims=z["rot"], base=1e6))
+        yarn = dict(att, rot=dict(dims=z["rot"], base=1e6, scaling=dict(factor=4.0, original=4096, fast=32.0, slow=1.0)))
+        delta = dict(heads=z["d_heads"], kv_heads=z["d_kv"], dim=z["d_dim"], vdim=z["d_vdim"], conv=z["taps"])
+        par = dict(left=yarn, right=dict(delta, kv_heads=z["d_heads"]), left_scale=0.6, right_scale=0.9)
+        P, D = SuvapelLayerConfig("parallel", par, dense), SuvapelLayerConfig("delta", delta, dense)
+        for label, layers in (("parallel x4", [P] * 4), ("delta x4", [D] * 4), ("hybrid (p, d, d, p)", [P, D, D, P])):
+            measure("suvapel " + label, name, lambda: SuvapelModel(SuvapelConfig(vocab, W, 1e-6, 0.3, z["side"], 1 << 24, layers), "bfloat16", dev))
+        gla = dict(heads=z["d_heads"], dim=z["d_dim"], vdim=z["d_vdim"], tau=16.0)
+        for label, layer in (("attention x4, dense", GutivikLayerConfig("attention", dict(att, v_mix=True), dense)),
+                             ("gla x4, dense", GutivikLayerConfig("gla", gla, dense))):
+            measure("gutivik " + label, name, lambda: GutivikModel(GutivikConfig(vocab, W, 1e-6, 1.0, 0.0, 1 << 24, [layer] * 4), "bfloat16", dev))
+        zpar = dict(left=dict(heads=z["heads"], kv_heads=z["kv_heads"], dim=z["dim"], vdim=z["dim"], scale=z["dim"] ** -0.5, q_temp=dict(coef=0.1, every=512)),
+                    right=dict(heads=z["d_heads"], dim=z["d_dim"], vdim=z["d_vdim"], decay=[0.99] * z["d_heads"], rot=dict(dims=z["d_dim"], base=1e4)))
+        zl = ZasazenLayerConfig("parallel", zpar, dict(kind="dense", ff=z["ff"] * 3 // 2))
+        measure("zasazen parallel x4, dense", name, lambda: ZasazenModel(ZasazenConfig(vocab, W, 1.0, 1e-6, None, 1 << 24, [zl] * 4), "bfloat16", dev))
+    print(json.dumps({"metric": "suvapel_throughput", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic", "layers": 4, "results": results}))
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--zasazen", default="", metavar="SIZES",
@@ -860,7 +910,10 @@ def main():
     ap.add_argument("--gutivik", default="", metavar="SIZES",
                     help="instead of the default workload: prefill / decode throughput of Gutivik stacks beside Retotar stacks of equal "
                          "width; comma-separated sizes of " + ", ".join(GUTIVIK_BENCH_SIZES))
-    ap.add_argument("--only", default="", metavar="TEXT", help="with --gutivik / --gaparax / --zasazen: only the stacks whose label contains TEXT (e.g. for a kernel trace of one model)")
+    ap.add_argument("--suvapel", default="", metavar="SIZES",
+                    help="instead of the default workload: prefill / decode throughput of Suvapel stacks beside Gutivik and Zasazen stacks of "
+                         "equal width; comma-separated sizes of " + ", ".join(SUVAPEL_BENCH_SIZES))
+    ap.add_argument("--only", default="", metavar="TEXT", help="with --gutivik / --gaparax / --zasazen / --suvapel: only the stacks whose label contains TEXT (e.g. for a kernel trace of one model)")
     ap.add_argument("--mixers", default="", metavar="SIZES",
                     help="instead of the default workload: prefill / decode throughput of the ragged-step engine's latent-attention + "
                          "state-space model beside the dense Llama-shaped stack of equal width; comma-separated sizes of " + ", ".join(SEQ_BENCH_SIZES))
@@ -908,6 +961,8 @@ def main():
         return bench_gaparax(args, dev)
     if args.zasazen:
         return bench_zasazen(args, dev)
+    if args.suvapel:
+        return bench_suvapel(args, dev)
     from zhilight_amd import ops  # noqa: F401  (raises if the HIP library is missing)
     from zhilight_amd.llama import LLaMA, ModelConfig, QuantConfig
 

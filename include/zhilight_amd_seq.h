@@ -320,19 +320,18 @@ int zls_lowrank_decay(const float* proj, int64_t ld, int64_t u_col0, int64_t low
 /* What a token needs before the recurrence.  Columns col0 .. of the fp32 rows proj[t] (ld) hold [q (kv_heads * dim) | k (kv_heads * dim) |
  * v (heads * vdim)] = C channels: each passes a causal convolution (w fp32 (C, taps), last column: the current token; inputs before a
  * portion from tail[slot] (taps - 1, C), which moves on; tail NULL when taps == 1) and SiLU; every q and k head is divided by
- * sqrt(sum of its squares + unit_eps), q also multiplied by q_scale.  Results: qkv fp32 (n_tok, C); qk fp32 (n_tok, kv_heads) = q . k of the
- * finished vectors; beta[t][h] = sigmoid(proj[t][b_col0 + h]); decay = exp(-rate[h] softplus(z + z_bias)) with z = z[t][z_col0 ..] (fp32
- * rows of ldz), one number per head (per_channel 0, decay fp32 (n_tok, heads)) or per head and key channel (decay (n_tok, heads * dim));
- * z_bias fp32, nullable, as many numbers.  dim <= 512. */
+ * sqrt(sum of its squares + unit_eps), q also multiplied by q_scale.  Results: qkv fp32 (n_tok, C); gates fp32 (n_tok, heads, 4) =
+ * (sigmoid(proj[t][b_col0 + h]), the decay of head h or 1, q . k of the finished vectors of the head's query / key head, 0).  The decay is
+ * exp(-rate[h] softplus(z + z_bias)) with z = z[t][z_col0 ..] (fp32 rows of ldz), one number per head (per_channel 0) or per head and key
+ * channel (then decay fp32 (n_tok, heads * dim)); z_bias fp32, nullable, as many numbers.  dim <= 512. */
 int zls_delta_prep(const float* proj, int64_t ld, int64_t col0, const float* w, float* tail, int64_t taps, int64_t heads, int64_t kv_heads,
                    int64_t dim, int64_t vdim, float q_scale, float unit_eps, int64_t b_col0, const float* z, int64_t ldz, int64_t z_col0,
-                   const float* z_bias, const float* rate, int per_channel, const zls_batch_t* b, float* qkv, float* qk, float* beta, float* decay,
-                   zl_stream_t s);
+                   const float* z_bias, const float* rate, int per_channel, const zls_batch_t* b, float* qkv, float* gates, float* decay, zl_stream_t s);
 /* Per head h (query / key head h / (heads / kv_heads)), tokens in order:  S <- g S (per key channel: row c of S by g[c]);
- * u = beta (v - S^T k);  S <- S + k u^T;  y[t][h] = S^T q.  Inputs as zls_delta_prep left them.  state fp32 (slots, heads, vdim, dim) --
+ * u = beta (v - S^T k);  S <- S + k u^T;  y[t][h] = S^T q.  Inputs as zls_delta_prep left them (decay NULL: one per head).  state fp32 (slots, heads, vdim, dim) --
  * the transpose of S, a value column's numbers side by side --, y fp32 (n_tok, heads * vdim).  dim <= 512. */
-int zls_delta_scan(const float* qkv, const float* qk, const float* beta, const float* decay, int per_channel, float* state, int64_t heads,
-                   int64_t kv_heads, int64_t dim, int64_t vdim, const zls_batch_t* b, float* y, zl_stream_t s);
+int zls_delta_scan(const float* qkv, const float* gates, const float* decay, float* state, int64_t heads, int64_t kv_heads, int64_t dim,
+                   int64_t vdim, const zls_batch_t* b, float* y, zl_stream_t s);
 
 /* ---- mixture of experts over a ragged step ------------------------------------------------------------------------------------------ */
 /* Router: s = softmax(logits[t]) over all n_out outputs (score_kind 0), sigmoid(logits[t][i]) of each (score_kind 1) or logits[t] (score_kind

@@ -19,8 +19,9 @@ BASE_FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-Wall", "-
 FLAGS = BASE_FLAGS + ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 # per-source extras.  w4_slab.hip: its item loops (up to 4 groups x 8 tiles, the next group's normalisation in slices between the
 # items) must unroll completely -- ring slots, accumulators and wait counts are static only then -- and the NORM instantiations
-# exceed the unroller's default budget for `#pragma unroll` (16 K): the ring went to scratch behind dynamic indices
-EXTRA_FLAGS = {"w4_slab.hip": ["-mllvm", "-pragma-unroll-threshold=200000"]}
+# exceed the unroller's default budget for `#pragma unroll` (16 K): the ring went to scratch behind dynamic indices.  csrc_seq/seq_gemm.hip: the
+# same for the accumulators of a 128 x 128 tile whose epilogue applies an activation to every one of them
+EXTRA_FLAGS = {"w4_slab.hip": ["-mllvm", "-pragma-unroll-threshold=200000"], "seq_gemm.hip": ["-mllvm", "-pragma-unroll-threshold=200000"]}
 
 
 # ZL_BUILD_EXPERIMENTAL=1: also build what was measured and left off the product path: the loader /
@@ -102,7 +103,7 @@ def build_seq(force=False, verbose=False):
         o = os.path.join(objdir, os.path.basename(src)[:-4] + ".o")
         objs.append(o)
         if force or _stale(o, [src] + deps):
-            jobs.append([HIPCC] + SEQ_FLAGS + ["-c", src, "-o", o])
+            jobs.append([HIPCC] + SEQ_FLAGS + EXTRA_FLAGS.get(os.path.basename(src), []) + ["-c", src, "-o", o])
 
     def run(cmd):
         if verbose:

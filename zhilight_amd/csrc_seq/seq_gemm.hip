@@ -10,7 +10,8 @@
 //               4 x 4 or 2 x 2 MFMA tiles of 16 x 16), 32-k slices of x and W staged through LDS (zero-filled past the edges), the next slice's global
 //               loads issued before the current slice's MFMAs.  bf16: v_mfma_f32_16x16x32_bf16; fp32: v_mfma_f32_16x16x4_f32.
 //               A long k with few output tiles is divided over workgroups (blockIdx.z), k_split_sum adds the parts.
-// Each has an instantiation with an epilogue (EPI: bias, activation, leading columns once more in the serving format).
+// Each has instantiations with an epilogue: EPI 1 adds a bias and writes leading columns once more in the serving format, EPI 2 also applies
+// an activation and a factor looked up per row.
 #include "seq_common.h"
 
 namespace {
@@ -41,12 +42,16 @@ struct GemmP {
     float* part; int k_part, n_parts;
 };
 
-template <int DT, int ODT, bool EPI>
+template <int DT, int ODT, int EPI>
 __device__ __forceinline__ void put(const GemmP& p, int row, int col, float v) {
-    if constexpr (EPI) {
+    if constexpr (EPI > 0) {
         if (p.bias) v += p.bias[col];
+    }
+    if constexpr (EPI == 2) {
         if (p.uact >= 0) v = unary_act(v, p.uact);
         if (p.f_table) v *= SeqT<DT>::ld(p.f_table, (size_t)min(max(p.f_rows[row], 0), p.f_n - 1) * p.f_ld + col);
+    }
+    if constexpr (EPI > 0) {
         if (col < p.n2) SeqT<DT>::st(p.y2, (size_t)row * p.ldy2 + col, v);
     }
     SeqT<ODT>::st(p.y, (size_t)row * p.ldy + col, v);
@@ -94,7 +99,7 @@ template <> struct Tile<ZL_F32> {
 // WT x WT MFMA tiles per wave: the workgroup's output tile is (32 WT) x (32 WT)
 // GATED: the weight rows come in blocks of 16 gate rows followed by their 16 up rows, so that a wave's even column tiles are gates and the
 // odd ones the up projections of the same 16 outputs; the epilogue writes act(gate, up) (gated_act: silu(gate) * up and others), half as many columns
-template <int DT, int ODT, int WT, bool GATED = false, bool EPI = false>
+template <int DT, int ODT, int WT, bool GATED = false, int EPI = 0>
 __global__ __launch_bounds__(256) void k_seq_gemm(const GemmP p) {
     typedef typename Tile<DT>::elem E;
     constexpr int RS = Tile<DT>::kRow;
@@ -211,7 +216,7 @@ __global__ __launch_bounds__(256) void k_seq_gemm(const GemmP p) {
 }
 
 // the parts of a k that was divided, added in order, and the epilogue
-template <int DT, int ODT, bool EPI>
+template <int DT, int ODT, int EPI>
 __global__ __launch_bounds__(256) void k_split_sum(const GemmP p) {
     const int64_t e = (int64_t)blockIdx.x * 256 + threadIdx.x, mn = (int64_t)p.m * p.n;
     if (e >= mn) return;
@@ -243,7 +248,7 @@ template <> struct Vec8<ZL_F32> {
 
 // CPW output columns per wave: the activation rows (L2) are read once per CPW weight rows (HBM) -- with 8 rows and one column per wave
 // the activations would be eight times the weight traffic
-template <int DT, int ODT, int MR, int CPW, bool EPI = false>
+template <int DT, int ODT, int MR, int CPW, int EPI = 0>
 __global__ __launch_bounds__(256) void k_seq_gemv(const GemmP p) {
     const int lane = threadIdx.x & 63;
     const int col0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * CPW;
@@ -301,7 +306,7 @@ __global__ __launch_bounds__(256) void k_seq_gemv(const GemmP p) {
 // activation row (B operand: lane = row; rows past m are zero), eight steps in flight, one v_mfma_f32_16x16x32_bf16 each.  The weights are
 // read exactly once, the activations cost half the weight bytes at 8 rows (L2), and no VALU multiply is spent.  The four partial tiles
 // meet in LDS.
-template <int ODT, bool EPI = false>
+template <int ODT, int EPI = 0>
 __global__ __launch_bounds__(256) void k_seq_gemv_mfma(const GemmP p) {
     __shared__ float red[4][16][17];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nrow = lane & 15, kq = lane >> 4;
@@ -374,7 +379,7 @@ __global__ __launch_bounds__(256) void k_seq_gemv_grouped(const GemmP p, const i
 }
 
 // 128 x 128 tiles (four times the MFMAs per LDS fragment) when they still fill the chip, 64 x 64 otherwise
-template <int DT, int ODT, bool EPI = false>
+template <int DT, int ODT, int EPI = 0>
 void launch_tiled(const GemmP& p, hipStream_t hs) {
     const int64_t big = (int64_t)((p.m + 127) / 128) * ((p.n + 127) / 128);
     if (p.part) {
@@ -390,7 +395,7 @@ void launch_tiled(const GemmP& p, hipStream_t hs) {
     }
 }
 
-template <int DT, int ODT, bool EPI = false>
+template <int DT, int ODT, int EPI = 0>
 int launch(const GemmP& p, hipStream_t hs) {
     if constexpr (DT == ZL_BF16) {
         if (!p.part && p.m >= 3 && p.m <= 16 && p.vec && (p.k & 7) == 0) {
@@ -438,9 +443,13 @@ extern "C" int zls_gemm_nt_act(const void* x, int64_t ldx, const void* w, const 
     const int64_t unit = dtype == ZL_BF16 ? 8 : 4;
     p.vec = (k % unit == 0 && ldx % unit == 0 && ((uintptr_t)x & 15) == 0 && ((uintptr_t)w & 15) == 0) ? 1 : 0;
     hipStream_t hs = (hipStream_t)s;
-    if (bias || act >= 0 || y2 || factor) {
-        if (dtype == ZL_BF16) return out_dtype == ZL_F32 ? launch<ZL_BF16, ZL_F32, true>(p, hs) : launch<ZL_BF16, ZL_BF16, true>(p, hs);
-        return launch<ZL_F32, ZL_F32, true>(p, hs);
+    if (act >= 0 || factor) {
+        if (dtype == ZL_BF16) return out_dtype == ZL_F32 ? launch<ZL_BF16, ZL_F32, 2>(p, hs) : launch<ZL_BF16, ZL_BF16, 2>(p, hs);
+        return launch<ZL_F32, ZL_F32, 2>(p, hs);
+    }
+    if (bias || y2) {
+        if (dtype == ZL_BF16) return out_dtype == ZL_F32 ? launch<ZL_BF16, ZL_F32, 1>(p, hs) : launch<ZL_BF16, ZL_BF16, 1>(p, hs);
+        return launch<ZL_F32, ZL_F32, 1>(p, hs);
     }
     if (dtype == ZL_BF16) return out_dtype == ZL_F32 ? launch<ZL_BF16, ZL_F32>(p, hs) : launch<ZL_BF16, ZL_BF16>(p, hs);
     return launch<ZL_F32, ZL_F32>(p, hs);

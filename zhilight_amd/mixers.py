@@ -847,9 +847,9 @@ class GatedDeltaRule:
         z = seqops.gemm_nt(lead, self.w_low) if self.w_low is not None else None               # fp32 [decay input | gate], the low-rank ones
         dec, dec0 = (z, 0) if self.per_channel else (proj, b0 + H)
         gate, gate0 = (z, H * d if self.per_channel else 0) if self.lowrank_gate else (proj, b0 + (H if self.per_channel else 2 * H))
-        qkv, qk, beta, decay = seqops.delta_prep(proj, col0, self.conv_w, self.tail, H, G, d, v, d ** -0.5, self.UNIT_EPS, b0, dec, dec0, self.dt_bias,
-                                                 self.rate, self.per_channel, batch)
-        y = seqops.delta_scan(qkv, qk, beta, decay, self.state, H, G, d, v, batch)
+        qkv, gates, decay = seqops.delta_prep(proj, col0, self.conv_w, self.tail, H, G, d, v, d ** -0.5, self.UNIT_EPS, b0, dec, dec0, self.dt_bias,
+                                               self.rate, self.per_channel, batch)
+        y = seqops.delta_scan(qkv, gates, decay, self.state, H, G, d, v, batch)
         return seqops.linear_attn_finish(y, False, 1.0, None, 0.0, H, v, H, self.norm_w, self.eps, gate, gate0, dtype, gate_act=self.gate_act, out=out,
                                          out_scale=out_scale)
 

@@ -799,7 +799,8 @@ def linear_attn_finish(y, norm_col, q_scale, m_vals, den_eps, heads, vdim, norm_
 
 # ---- gated delta rule --------------------------------------------------------------------------------------------------------------------
 def delta_prep(proj, col0, conv_w, tail, heads, kv_heads, dim, vdim, q_scale, unit_eps, b_col0, z, z_col0, z_bias, rate, per_channel, batch):
-    """convolution + SiLU, unit vectors, q . k, beta and decays of a step: (qkv, qk, beta, decay) for delta_scan; the carried tail moves on"""
+    """convolution + SiLU, unit vectors, gates and decays of a step: (qkv, gates, decay) for delta_scan -- gates (n_tok, heads, 4) holds beta, the
+    decay per head (1 when it is per channel) and q . k, decay (n_tok, heads * dim) or None --; the carried tail moves on"""
     _cuda(proj, conv_w, tail, z, z_bias, rate)
     _f32(proj, conv_w, tail, z, z_bias, rate)
     channels, taps = conv_w.shape
@@ -809,27 +810,25 @@ def delta_prep(proj, col0, conv_w, tail, heads, kv_heads, dim, vdim, q_scale, un
     if rate.numel() != heads or (z_bias is not None and z_bias.numel() != D) or z.shape[0] != proj.shape[0] or proj.shape[0] != batch.n_tok:
         raise ZLError("delta_prep: shapes")
     n, dev = batch.n_tok, proj.device
-    qkv, qk = torch.empty((n, channels), dtype=torch.float32, device=dev), torch.empty((n, kv_heads), dtype=torch.float32, device=dev)
-    beta, decay = torch.empty((n, heads), dtype=torch.float32, device=dev), torch.empty((n, D), dtype=torch.float32, device=dev)
+    qkv, gates = torch.empty((n, channels), dtype=torch.float32, device=dev), torch.empty((n, heads, 4), dtype=torch.float32, device=dev)
+    decay = torch.empty((n, D), dtype=torch.float32, device=dev) if per_channel else None
     check(lib().zls_delta_prep(_p(proj), _i(proj.shape[1]), _i(col0), _p(conv_w), _p(tail), _i(taps), _i(heads), _i(kv_heads), _i(dim), _i(vdim),
                                _f(q_scale), _f(unit_eps), _i(b_col0), _p(z), _i(z.shape[1]), _i(z_col0), _p(z_bias), _p(rate),
-                               C.c_int(int(per_channel)), batch.ref, _p(qkv), _p(qk), _p(beta), _p(decay), _stream()), "delta_prep")
-    return qkv, qk, beta, decay
+                               C.c_int(int(per_channel)), batch.ref, _p(qkv), _p(gates), _p(decay), _stream()), "delta_prep")
+    return qkv, gates, decay
 
 
-def delta_scan(qkv, qk, beta, decay, state, heads, kv_heads, dim, vdim, batch):
+def delta_scan(qkv, gates, decay, state, heads, kv_heads, dim, vdim, batch):
     """S <- g S; u = beta (v - S^T k); S <- S + k u^T; y = S^T q over the step's portions: fp32 y (n_tok, heads * vdim); state (slots, heads,
-    vdim, dim) moves on.  decay (n_tok, heads) or, per key channel, (n_tok, heads * dim)"""
-    _cuda(qkv, qk, beta, decay, state)
-    _f32(qkv, qk, beta, decay, state)
+    vdim, dim) moves on.  Inputs from delta_prep"""
+    _cuda(qkv, gates, decay, state)
+    _f32(qkv, gates, decay, state)
     n = batch.n_tok
-    per_channel = decay.shape[1] == heads * dim and dim > 1
-    if tuple(qkv.shape) != (n, 2 * kv_heads * dim + heads * vdim) or tuple(qk.shape) != (n, kv_heads) or tuple(beta.shape) != (n, heads) or \
-            tuple(decay.shape) != (n, heads * dim if per_channel else heads) or tuple(state.shape[1:]) != (heads, vdim, dim):
+    if tuple(qkv.shape) != (n, 2 * kv_heads * dim + heads * vdim) or tuple(gates.shape) != (n, heads, 4) or \
+            (decay is not None and tuple(decay.shape) != (n, heads * dim)) or tuple(state.shape[1:]) != (heads, vdim, dim):
         raise ZLError("delta_scan: shapes")
     y = torch.empty((n, heads * vdim), dtype=torch.float32, device=qkv.device)
-    check(lib().zls_delta_scan(_p(qkv), _p(qk), _p(beta), _p(decay), C.c_int(int(per_channel)), _p(state), _i(heads), _i(kv_heads), _i(dim),
-                               _i(vdim), batch.ref, _p(y), _stream()), "delta_scan")
+    check(lib().zls_delta_scan(_p(qkv), _p(gates), _p(decay), _p(state), _i(heads), _i(kv_heads), _i(dim), _i(vdim), batch.ref, _p(y), _stream()), "delta_scan")
     return y
 
 
