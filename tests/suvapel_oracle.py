@@ -190,3 +190,79 @@ def forward(tokens, weights, cfg, keep=None):
         if keep is not None:
             keep.append(x.clone())
     return model_norm(x, weights, "final.norm") @ _w(weights, "head").T
+
+
+# ---- test weights ------------------------------------------------------------------------------------------------------------------------
+def random_weights(cfg, seed=0):
+    """every tensor the configuration asks for, bf16-representable values (both serving formats start from the same numbers).  Key
+    projections lean towards the query projections: a sequence's first delta-rule output is (q . k) v over its own root mean square, whose
+    SIGN hangs on a product that random matrices let come close to zero."""
+    g = torch.Generator().manual_seed(seed)
+    W, sd = cfg["width"], {}
+
+    def mat(name, rows, cols, std=None):
+        sd[name] = (torch.randn(rows, cols, generator=g) * (std if std is not None else cols ** -0.5)).to(torch.bfloat16)
+
+    def vec(name, n, std=0.2, mean=0.0):
+        sd[name] = (mean + std * torch.randn(n, generator=g)).to(torch.bfloat16)
+
+    def norm(name):
+        vec(name, W, 0.2, 1.0)
+        vec(name + ".b", W, 0.2)
+        sd[name + ".alpha"] = torch.tensor(0.4 + 0.4 * float(torch.rand(1, generator=g))).to(torch.bfloat16)
+
+    def conv(name, rows, taps):
+        sd[name] = (0.4 * torch.randn(rows, taps, generator=g)).to(torch.bfloat16)
+        sd[name][:, -1] += 0.7
+
+    def delta(p, m, per_channel):
+        H, G, d, e, low = m["heads"], m["kv_heads"], m["dim"], m["vdim"], m.get("low", 10)
+        for n, rows in (("q", G * d), ("k", G * d), ("v", H * e)):
+            mat(p + n, rows, W, 1.5 * W ** -0.5)
+            conv(p + n + ".conv", rows, m["conv"])
+        sd[p + "k"] = (0.8 * sd[p + "q"].float() + 0.6 * sd[p + "k"].float()).to(torch.bfloat16)
+        mat(p + "b", H, W)
+        sd[p + "A_log"] = (torch.rand(H, generator=g) * 2.5 - 1.5).to(torch.bfloat16)
+        vec(p + "norm", e, 0.2, 1.0)
+        if per_channel:
+            mat(p + "a1", low, W)
+            mat(p + "a2", H * d, low)
+            vec(p + "dt_bias", H * d, 1.2, -3.0)
+            mat(p + "g1", low, W)
+            mat(p + "g2", H * e, low)
+        else:
+            mat(p + "a", H, W)
+            vec(p + "dt_bias", H, 1.0, -3.0)
+            mat(p + "g", H * e, W)
+        mat(p + "o", W, H * e)
+
+    mat("embed", cfg["vocab"], W, 1.0)
+    mat("side.embed", cfg["vocab"], len(cfg["layers"]) * cfg["token_side"]["dim"], 1.0)
+    mat("head", cfg["vocab"], W)
+    norm("final.norm")
+    for i, l in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", l["mixer"]
+        norm(p + "norm1")
+        if l["type"] == "delta":
+            delta(p + "mix.", m, False)
+        else:
+            a = m["left"]
+            H, G, d, e = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
+            for n, rows in (("q", H * d), ("k", G * d), ("v", G * e)):
+                mat(p + "mix.left." + n, rows, W)
+                conv(p + "mix.left." + n + ".conv", rows, a["conv"])
+            mat(p + "mix.left.g", H, W)
+            mat(p + "mix.left.o", W, H * e)
+            delta(p + "mix.right.", m["right"], True)
+        if l.get("mlp") is not None:
+            ff = l["mlp"]["ff"]
+            for n in ("gate", "up"):
+                mat(p + "mlp." + n, ff, W)
+                vec(p + "mlp." + n + ".b", ff, 0.3)
+            mat(p + "mlp.down", W, ff)
+            vec(p + "mlp.down.b", W, 0.3)
+        dim = cfg["token_side"]["dim"]
+        mat(p + "side.gate", dim, W)
+        mat(p + "side.proj", W, dim)
+        vec(p + "side.norm", W, 0.2, 1.0)
+    return sd
