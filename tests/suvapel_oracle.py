@@ -195,7 +195,7 @@ def forward(tokens, weights, cfg, keep=None):
 # ---- test weights ------------------------------------------------------------------------------------------------------------------------
 def random_weights(cfg, seed=0):
     """every tensor the configuration asks for, bf16-representable values (both serving formats start from the same numbers).  Key
-    projections lean towards the query projections: a sequence's first delta-rule output is (q . k) v over its own root mean square, whose
+    projections and convolutions lean towards the queries': a sequence's first delta-rule output is (q . k) v over its own root mean square, whose
     SIGN hangs on a product that random matrices let come close to zero."""
     g = torch.Generator().manual_seed(seed)
     W, sd = cfg["width"], {}
@@ -220,7 +220,8 @@ def random_weights(cfg, seed=0):
         for n, rows in (("q", G * d), ("k", G * d), ("v", H * e)):
             mat(p + n, rows, W, 1.5 * W ** -0.5)
             conv(p + n + ".conv", rows, m["conv"])
-        sd[p + "k"] = (0.8 * sd[p + "q"].float() + 0.6 * sd[p + "k"].float()).to(torch.bfloat16)
+        sd[p + "k"] = (0.9 * sd[p + "q"].float() + 0.4 * sd[p + "k"].float()).to(torch.bfloat16)
+        sd[p + "k.conv"] = (sd[p + "q.conv"].float() + 0.2 * sd[p + "k.conv"].float()).to(torch.bfloat16)
         mat(p + "b", H, W)
         sd[p + "A_log"] = (torch.rand(H, generator=g) * 2.5 - 1.5).to(torch.bfloat16)
         vec(p + "norm", e, 0.2, 1.0)

@@ -75,13 +75,14 @@ def cfg_a():
                       delta_l(heads=3, kv_heads=3, dim=40, vdim=36, conv=3, ff=None)])
 
 
-def cfg_odd(vdim=1):
+def cfg_odd(one=1):
     """sizes no matrix-core kernel and no 16-byte access takes, and values that a particular model may make equal or 1: one head, heads = kv
     heads, one tap, a window of one key, no kept keys, all of a head rotated, key and value sizes that differ by one, ranks of 1 and 3,
-    scales and multipliers of 1, one column of side input; values of one number (whose norm is their sign: for fp32)"""
-    return model_cfg([parallel_l(attn_m(heads=3, kv_heads=3, dim=10, vdim=7, conv=1, size=1, keep=0, dims=10, factor=1.0), delta_m(heads=1, kv_heads=1, dim=5, vdim=3, conv=1, low=1), 1.0, 1.0, ff=33),
-                      delta_l(heads=5, kv_heads=1, dim=9, vdim=10, conv=6, ff=17), delta_l(heads=2, kv_heads=2, dim=33, vdim=vdim, conv=2, ff=None),
-                      parallel_l(attn_m(heads=5, kv_heads=1, dim=14, vdim=9, conv=2, size=65, keep=70, dims=2, fast=3.0), delta_m(heads=6, kv_heads=3, dim=1, vdim=18, conv=5, low=3), -0.5, 2.0, ff=None)],
+    scales and multipliers of 1, one column of side input; keys and values of `one` number (a unit vector or norm of one number is
+    its sign, which rounding may flip near 0: 1 is for fp32)"""
+    return model_cfg([parallel_l(attn_m(heads=3, kv_heads=3, dim=10, vdim=7, conv=1, size=1, keep=0, dims=10, factor=1.0), delta_m(heads=1, kv_heads=1, dim=5, vdim=3 * one, conv=1, low=1), 1.0, 1.0, ff=33),
+                      delta_l(heads=5, kv_heads=1, dim=9, vdim=10, conv=6, ff=17), delta_l(heads=2, kv_heads=2, dim=33, vdim=one, conv=2, ff=None),
+                      parallel_l(attn_m(heads=5, kv_heads=1, dim=14, vdim=9, conv=2, size=65, keep=70, dims=2, fast=3.0), delta_m(heads=6, kv_heads=3, dim=one, vdim=18, conv=5, low=3), -0.5, 2.0, ff=None)],
                      width=70, vocab=90, mult=1.0, side=1)
 
 
@@ -537,7 +538,7 @@ def test_same_bits_after_pages_and_slots_were_used_by_others(dev):
 @pytest.mark.parametrize("dtype", DTYPES)
 def test_odd_sizes_whole_in_portions_and_decoded(dev, dtype):
     cfg = cfg_odd(1 if dtype == torch.float32 else 6)
-    sd = O.random_weights(cfg, 25)
+    sd = O.random_weights(cfg, 27)
     toks = tokens_of(cfg, 140, 26)
     logits = O.forward(toks, sd, cfg)
     eng = make(cfg, sd, dtype, dev)

@@ -9,6 +9,7 @@
 //               own: NGL neighbouring lanes hold a column, NPT numbers each, and meet in two DPP butterflies per token.  With a = g S the
 //               token needs only the sums a.k and a.q at once:  u = beta (v - a.k),  S = a + k u,  o = a.q + (q.k) u.
 //               The state lies (head, column, key coordinate), so a lane's numbers are 16-byte runs.
+// k_delta_step  the same for a step of single tokens, without staging
 // All of it is fp32 in both serving formats.
 #include "seq_common.h"
 
@@ -208,6 +209,16 @@ template <int CTRL>
 __device__ __forceinline__ float dpp_add(float v) {
     return v + __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, 0xf, 0xf, true));
 }
+// every lane plus the lane 16 / 32 further on: the swap instructions exchange odd rows (upper halves) of one register with even rows (lower
+// halves) of the other, so two copies of v come out as the two addends
+__device__ __forceinline__ float rows_add(float v) {
+    const auto r = __builtin_amdgcn_permlane16_swap(__builtin_bit_cast(uint32_t, v), __builtin_bit_cast(uint32_t, v), false, false);
+    return __builtin_bit_cast(float, (uint32_t)r[0]) + __builtin_bit_cast(float, (uint32_t)r[1]);
+}
+__device__ __forceinline__ float halves_add(float v) {
+    const auto r = __builtin_amdgcn_permlane32_swap(__builtin_bit_cast(uint32_t, v), __builtin_bit_cast(uint32_t, v), false, false);
+    return __builtin_bit_cast(float, (uint32_t)r[0]) + __builtin_bit_cast(float, (uint32_t)r[1]);
+}
 // two sums over NGL neighbouring lanes, in every lane: quads by permutation (xor 1, xor 2), then mirrored halves and rows of 16
 template <int NGL>
 __device__ __forceinline__ void group_sums(float& a, float& b) {
@@ -215,8 +226,8 @@ __device__ __forceinline__ void group_sums(float& a, float& b) {
     a = dpp_add<0x4E>(a); b = dpp_add<0x4E>(b);
     if constexpr (NGL >= 8) { a = dpp_add<0x141>(a); b = dpp_add<0x141>(b); }
     if constexpr (NGL >= 16) { a = dpp_add<0x140>(a); b = dpp_add<0x140>(b); }
-    if constexpr (NGL >= 32) { a += __shfl_xor(a, 16, 64); b += __shfl_xor(b, 16, 64); }
-    if constexpr (NGL >= 64) { a += __shfl_xor(a, 32, 64); b += __shfl_xor(b, 32, 64); }
+    if constexpr (NGL >= 32) { a = rows_add(a); b = rows_add(b); }
+    if constexpr (NGL >= 64) { a = halves_add(a); b = halves_add(b); }
 }
 
 __device__ __forceinline__ float4 load4(const float* p, int n, int vec) {      // up to 4 numbers, n of them there
@@ -424,6 +435,59 @@ __global__ __launch_bounds__(kScanT) void k_delta_scan(const DeltaP p, const zls
     }
 }
 
+// A step in which every portion is ONE token: the state is the traffic.  Nothing is staged -- a lane reads its numbers of the state, the
+// token's key, query and decays straight from memory, all loads in flight together, and writes its numbers of the state back.
+template <int NGL, int NPT, bool PC>
+__global__ __launch_bounds__(256) void k_delta_step(const DeltaP p, const zls_batch_t b) {
+    constexpr int F = NPT / 4;
+    const int g = threadIdx.x % NGL, sq = blockIdx.x, h = blockIdx.y, hk = h / (p.heads / p.kv_heads), col = blockIdx.z * (256 / NGL) + threadIdx.x / NGL;
+    const int d = p.dim, P = p.vdim, H = p.heads, qk_dim = p.kv_heads * d, C = 2 * qk_dim + H * P;
+    const size_t t = b.seq_start[sq];
+    const bool ok = col < P;
+    float* st = p.state + (((size_t)b.seq_slot[sq] * H + h) * P + (ok ? col : 0)) * d;
+    const float* row = p.qkv + t * C + hk * d;
+    const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+    float4 s[F], k[F], q[F], a[F];
+    const float4 sc = *reinterpret_cast<const float4*>(p.gates + (t * H + h) * 4);
+#pragma unroll
+    for (int f = 0; f < F; ++f) {
+        const int n = 4 * (g + NGL * f);
+        s[f] = k[f] = q[f] = zero;
+        a[f] = make_float4(sc.y, sc.y, sc.y, sc.y);
+        if (n < d) {
+            s[f] = load4(st + n, d - n, p.vec);
+            k[f] = load4(row + qk_dim + n, d - n, p.vec);
+            q[f] = load4(row + n, d - n, p.vec);
+            if constexpr (PC) a[f] = load4(p.decay + (t * H + h) * d + n, d - n, p.vec);
+        }
+    }
+    const float v = ok ? p.qkv[t * C + 2 * qk_dim + h * P + col] : 0.f;
+    float dk = 0.f, dq = 0.f;
+#pragma unroll
+    for (int f = 0; f < F; ++f) {
+        s[f].x *= a[f].x; s[f].y *= a[f].y; s[f].z *= a[f].z; s[f].w *= a[f].w;
+        dk = fmaf(s[f].x, k[f].x, dk); dk = fmaf(s[f].y, k[f].y, dk); dk = fmaf(s[f].z, k[f].z, dk); dk = fmaf(s[f].w, k[f].w, dk);
+        dq = fmaf(s[f].x, q[f].x, dq); dq = fmaf(s[f].y, q[f].y, dq); dq = fmaf(s[f].z, q[f].z, dq); dq = fmaf(s[f].w, q[f].w, dq);
+    }
+    group_sums<NGL>(dk, dq);
+    const float u = sc.x * (v - dk);
+    if (!ok) return;
+    if (g == 0) p.y[(t * H + h) * P + col] = fmaf(sc.z, u, dq);
+#pragma unroll
+    for (int f = 0; f < F; ++f) {
+        const int n = 4 * (g + NGL * f);
+        if (n >= d) continue;
+        const float r[4] = {fmaf(k[f].x, u, s[f].x), fmaf(k[f].y, u, s[f].y), fmaf(k[f].z, u, s[f].z), fmaf(k[f].w, u, s[f].w)};
+        if (p.vec) {
+            *reinterpret_cast<float4*>(st + n) = make_float4(r[0], r[1], r[2], r[3]);
+        } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+                if (n + e < d) st[n + e] = r[e];
+        }
+    }
+}
+
 }  // namespace
 
 extern "C" int zls_delta_prep(const float* proj, int64_t ld, int64_t col0, const float* w, float* tail, int64_t taps, int64_t heads, int64_t kv_heads,
@@ -470,13 +534,29 @@ extern "C" int zls_delta_scan(const float* qkv, const float* gates, const float*
     p.dim = (int)dim; p.vdim = (int)vdim;
     p.vec = (dim % 4 == 0 && C % 4 == 0 && al(qkv) && al(state) && (!decay || al(decay))) ? 1 : 0;
     const int ngl = dim <= 16 ? 4 : dim <= 32 ? 8 : dim <= 128 ? 16 : dim <= 256 ? 32 : 64;
+    hipStream_t hs = (hipStream_t)s;
+    if (b->max_count == 1) {
+        const int64_t parts = (vdim * ngl + 255) / 256;
+        ZL_CHECK_ARG(parts <= 65535, ZL_ELIMIT);
+        const dim3 grid((unsigned)b->n_seq, (unsigned)heads, (unsigned)parts);
+#define STEP(NGL, NPT)                                                                                         \
+    if (decay) hipLaunchKernelGGL((k_delta_step<NGL, NPT, true>), grid, dim3(256), 0, hs, p, *b);              \
+    else hipLaunchKernelGGL((k_delta_step<NGL, NPT, false>), grid, dim3(256), 0, hs, p, *b)
+        if (dim <= 16) { STEP(4, 4); }
+        else if (dim <= 32) { STEP(8, 4); }
+        else if (dim <= 64) { STEP(16, 4); }
+        else if (dim <= 128) { STEP(16, 8); }
+        else if (dim <= 256) { STEP(32, 8); }
+        else { STEP(64, 8); }
+#undef STEP
+        return zl_launch_status();
+    }
     // two columns per group of lanes once single ones fill the chip's 1024 SIMDs
     const int64_t waves = (int64_t)b->n_seq * heads * ((vdim * ngl + 63) / 64);
     const int cpl = waves > 1024 && vdim * ngl > kScanT ? 2 : 1, cols = kScanT / ngl * cpl;
     const int64_t parts = (vdim + cols - 1) / cols;
     ZL_CHECK_ARG(parts <= 65535 && heads * vdim * 64 < (1LL << 31), ZL_ELIMIT);
     const dim3 grid((unsigned)b->n_seq, (unsigned)heads, (unsigned)parts);
-    hipStream_t hs = (hipStream_t)s;
 #define GO(NGL, NPT, CPL, PC) hipLaunchKernelGGL((k_delta_scan<NGL, NPT, CPL, PC>), grid, dim3(kScanT), 0, hs, p, *b)
 #define SIZES(NGL, NPT)                                                                 \
     if (cpl == 2) { if (decay) GO(NGL, NPT, 2, true); else GO(NGL, NPT, 2, false); }    \

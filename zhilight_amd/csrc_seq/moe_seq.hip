@@ -197,7 +197,7 @@ template <int DT>
 __global__ __launch_bounds__(256) void k_act_mul(const float* __restrict__ gu, int64_t ld, int ff, int kind, float alpha, float limit, int block,
                                                  void* __restrict__ out, int64_t ldo) {
     const size_t r = blockIdx.x;
-    for (int c = threadIdx.x; c < ff; c += 256) {
+    for (int c = blockIdx.y * 256 + threadIdx.x; c < ff; c += gridDim.y * 256) {
         const int gi = block > 0 ? (c / block) * 2 * block + c % block : c, ui = block > 0 ? gi + block : ff + c;
         SeqT<DT>::st(out, r * ldo + c, gated_act(gu[r * ld + gi], gu[r * ld + ui], kind, alpha, limit));
     }
@@ -260,7 +260,9 @@ extern "C" int zls_silu_mul(const float* gu, int64_t rows, int64_t ff, void* out
 extern "C" int zls_act_mul(const float* gu, int64_t ld, int64_t rows, int64_t ff, int kind, float alpha, float limit, int64_t block, void* out, int64_t ldo, int dtype,
                            zl_stream_t s) {
     ZL_CHECK_ARG(gu && out && rows > 0 && ff > 0 && kind >= 0 && kind <= 2 && block >= 0 && (block == 0 || ff % block == 0) && ld >= 2 * ff && ldo >= ff, ZL_EINVAL);
-#define CALL(DT) hipLaunchKernelGGL((k_act_mul<DT>), dim3((unsigned)rows), dim3(256), 0, (hipStream_t)s, gu, ld, (int)ff, kind, alpha, limit, (int)block, out, ldo);
+    const int64_t want = rows >= 512 ? 1 : (ff + 255) / 256;               // (few rows: a row over several workgroups)
+    const unsigned parts = (unsigned)(want < 64 ? want : 64);
+#define CALL(DT) hipLaunchKernelGGL((k_act_mul<DT>), dim3((unsigned)rows, parts), dim3(256), 0, (hipStream_t)s, gu, ld, (int)ff, kind, alpha, limit, (int)block, out, ldo);
     ZLS_DISPATCH(dtype, CALL)
 #undef CALL
     return zl_launch_status();
