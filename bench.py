@@ -881,10 +881,10 @@ def bench_suvapel(args, dev):
                    mask=dict(size=z["window"], keep_first=z["keep"]), rot=dict(dims=z["rot"], base=1e6))
         yarn = dict(att, rot=dict(dims=z["rot"], base=1e6, scaling=dict(factor=4.0, original=4096, fast=32.0, slow=1.0)))
         delta = dict(heads=z["d_heads"], kv_heads=z["d_kv"], dim=z["d_dim"], vdim=z["d_vdim"], conv=z["taps"])
-        par = dict(left=yarn, right=dict(delta, kv_heads=z["d_heads"]), left_scale=0.6, right_scale=0.9)
+        par = dict(left=yarn, right=dict(delta, kv_heads=z["d_heads"]), left_scale=0.7, right_scale=0.8)
         P, D = SuvapelLayerConfig("parallel", par, dense), SuvapelLayerConfig("delta", delta, dense)
         for label, layers in (("parallel x4", [P] * 4), ("delta x4", [D] * 4), ("hybrid (p, d, d, p)", [P, D, D, P])):
-            measure("suvapel " + label, name, lambda: SuvapelModel(SuvapelConfig(vocab, W, 1e-6, 0.3, z["side"], 1 << 24, layers), "bfloat16", dev))
+            measure("suvapel " + label, name, lambda: SuvapelModel(SuvapelConfig(vocab, W, 1e-6, 0.4, z["side"], 1 << 24, layers), "bfloat16", dev))
         gla = dict(heads=z["d_heads"], dim=z["d_dim"], vdim=z["d_vdim"], tau=16.0)
         for label, layer in (("attention x4, dense", GutivikLayerConfig("attention", dict(att, v_mix=True), dense)),
                              ("gla x4, dense", GutivikLayerConfig("gla", gla, dense))):
